@@ -1,8 +1,8 @@
-// Layer norm with a weight and no shift, fused with what surrounds it, and the start of a
-// residual stream with learned positions:
+// Layer norm with a weight (and optionally a shift), fused with what surrounds it, and the start of
+// a residual stream with learned positions:
 //   sm_layer_norm  the fp32 residual row takes a sublayer's output times a constant in place,
 //                  x += mult * y (y in the model dtype; optional), and the same workgroup stores
-//                  LN(x) * w = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w rounded to the
+//                  LN(x) * w = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w (+ b) rounded to the
 //                  output dtype (optional: without w only the stream moves on).
 //   sm_embed_pos   x[t] = table[token[t]] + pos_table[position[t]], summed in fp32.
 // One workgroup of four waves per row.  The new row is kept in LDS between the passes (sum,
@@ -22,7 +22,8 @@ constexpr int kThreads = 256;
 template <typename TY, typename TO, bool VEC>
 __global__ void __launch_bounds__(kThreads)
 layer_norm_kernel(float* __restrict__ x, const TY* __restrict__ y, float mult,
-                  const float* __restrict__ w, TO* __restrict__ out, int W, float eps) {
+                  const float* __restrict__ w, const float* __restrict__ b, TO* __restrict__ out,
+                  int W, float eps) {
   extern __shared__ float s_row[];
   __shared__ float s_red[kThreads / 64];
   constexpr int V = VEC ? 4 : 1;
@@ -69,9 +70,14 @@ layer_norm_kernel(float* __restrict__ x, const TY* __restrict__ y, float mult,
       load4<float>(w + c, ww);
 #pragma unroll
       for (int e = 0; e < 4; ++e) v[e] = (v[e] - mean) * inv * ww[e];
+      if (b != nullptr) {
+        load4<float>(b + c, ww);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] += ww[e];
+      }
       store4<TO>(out + base + c, v);
     } else {
-      out[base + c] = from_f32<TO>((s_row[c] - mean) * inv * w[c]);
+      out[base + c] = from_f32<TO>((s_row[c] - mean) * inv * w[c] + (b != nullptr ? b[c] : 0.f));
     }
   }
 }
@@ -109,21 +115,22 @@ embed_pos_kernel(const T* __restrict__ table, const T* __restrict__ pos_table,
 extern "C" {
 
 // x fp32 [rows, W] contiguous (updated in place when y is given); y (nullable) [rows, W] in dtype
-// dt_y; w (nullable) fp32 [W]; out (with w) [rows, W] in dtype dt_out.  W * 4 bytes of LDS.
+// dt_y; w (nullable) fp32 [W]; b (nullable) fp32 [W]; out (with w) [rows, W] in dtype dt_out.  W * 4 bytes of LDS.
 hipError_t sm_layer_norm(int dt_y, int dt_out, float* x, const void* y, float mult,
-                         const float* w, void* out, int rows, int W, float eps, hipStream_t st) {
+                         const float* w, const float* b, void* out, int rows, int W, float eps,
+                         hipStream_t st) {
   if (rows == 0 || (!y && !w)) return hipSuccess;
   if (W < 1 || (size_t)W * sizeof(float) > 65536 - 64 || (w && !out)) return hipErrorInvalidValue;
   const size_t lds = (size_t)W * sizeof(float);
   const bool vec = W % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0 &&
-                   (uintptr_t)w % 16 == 0 && (uintptr_t)out % 16 == 0;
+                   (uintptr_t)w % 16 == 0 && (uintptr_t)b % 16 == 0 && (uintptr_t)out % 16 == 0;
 #define CALL_Y(TY, TO)                                                                          \
   {                                                                                             \
     if (vec)                                                                                    \
-      layer_norm_kernel<TY, TO, true><<<rows, kThreads, lds, st>>>(x, (const TY*)y, mult, w,    \
+      layer_norm_kernel<TY, TO, true><<<rows, kThreads, lds, st>>>(x, (const TY*)y, mult, w, b, \
                                                                    (TO*)out, W, eps);           \
     else                                                                                        \
-      layer_norm_kernel<TY, TO, false><<<rows, kThreads, lds, st>>>(x, (const TY*)y, mult, w,   \
+      layer_norm_kernel<TY, TO, false><<<rows, kThreads, lds, st>>>(x, (const TY*)y, mult, w, b, \
                                                                     (TO*)out, W, eps);          \
   }
 #define CALL_O(TO)                                    \

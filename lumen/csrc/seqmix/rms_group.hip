@@ -7,6 +7,11 @@
 //                  dtype (the input of the next sublayer's GEMMs).
 //   sm_gate_rows   out[t, d] = gelu_tanh(z[t, d]) * table[token[t], col0 + d]: a slice of a
 //                  per-token embedding row gated by a projection of the stream.
+//   sm_gated_rms   the read-out of a recurrence: the fp32 row, its group RMS norm and a gate from the
+//                  layer's projection, stored in the model dtype.  The gate multiplies before the
+//                  norm (x * act(g), then normed, times w) or after it (normed, times w, times
+//                  act(g)); act is SiLU or the sigmoid; w is one weight per channel or one per
+//                  group entry shared by the groups.
 // One workgroup of four waves per row.  With four or more groups a wave owns a group (and walks
 // the groups four at a time); with fewer, 4 / groups waves share one and add their partial sums in
 // a fixed order, so the result never depends on timing.  Sums, roots and products are fp32.
@@ -82,6 +87,74 @@ group_rms_kernel(const TI* __restrict__ x, long long ldx, const float* __restric
   }
 }
 
+// the row (gated, when the gate comes first) stays in LDS between the two passes; groups are dealt
+// out to the waves as above
+template <typename T, bool VEC>
+__global__ void __launch_bounds__(256)
+gated_rms_kernel(const float* __restrict__ x, const T* __restrict__ g, long long ldg,
+                 const float* __restrict__ w, T* __restrict__ out, int W, int groups, int shared_w,
+                 int gate_first, int sigmoid, float eps) {
+  extern __shared__ float s_row[];
+  __shared__ float s_part[4];
+  const int r = blockIdx.x, lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+  const int gs = W / groups;
+  const int wpg = groups >= 4 ? 1 : groups == 1 ? 4 : groups == 2 ? 2 : 1;   // waves per group
+  const int per_pass = 4 / wpg;
+  const int slot = wv / wpg, sub = wv % wpg;
+  const float* xr = x + (long long)r * W;
+  const T* gr = g + (long long)r * ldg;
+  T* orow = out + (long long)r * W;
+  constexpr int V = VEC ? 4 : 1;
+  for (int g0 = 0; g0 < groups; g0 += per_pass) {
+    const int gi = g0 + slot;
+    const bool on = gi < groups && slot < per_pass;
+    float ss = 0.f;
+    if (on) {
+      for (int c = (sub * 64 + lane) * V; c < gs; c += wpg * 64 * V) {
+        const int col = gi * gs + c;
+        float v[V], z[V];
+        if constexpr (VEC) load4<float>(xr + col, v);
+        else v[0] = xr[col];
+        if (gate_first) {
+          if constexpr (VEC) load4<T>(gr + col, z);
+          else z[0] = to_f32(gr[col]);
+#pragma unroll
+          for (int e = 0; e < V; ++e) v[e] *= sigmoid ? sigmoid_f(z[e]) : silu_f(z[e]);
+        }
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          ss += v[e] * v[e];
+          s_row[col + e] = v[e];
+        }
+      }
+    }
+    ss = wave_sum(ss);
+    if (lane == 0) s_part[wv] = ss;
+    __syncthreads();
+    if (on) {
+      float tot = 0.f;
+      for (int k = 0; k < wpg; ++k) tot += s_part[slot * wpg + k];
+      const float inv = 1.f / sqrtf(tot / (float)gs + eps);
+      for (int c = (sub * 64 + lane) * V; c < gs; c += wpg * 64 * V) {   // its own entries again
+        const int col = gi * gs + c;
+        const float* wp = w + (shared_w ? c : col);
+        float v[V], z[V];
+#pragma unroll
+        for (int e = 0; e < V; ++e) v[e] = s_row[col + e] * inv * wp[e];
+        if (!gate_first) {
+          if constexpr (VEC) load4<T>(gr + col, z);
+          else z[0] = to_f32(gr[col]);
+#pragma unroll
+          for (int e = 0; e < V; ++e) v[e] *= sigmoid ? sigmoid_f(z[e]) : silu_f(z[e]);
+        }
+        if constexpr (VEC) store4<T>(orow + col, v);
+        else orow[col] = from_f32<T>(v[0]);
+      }
+    }
+    __syncthreads();
+  }
+}
+
 template <typename T>
 __global__ void gate_rows_kernel(const T* __restrict__ z, long long ldz, const T* __restrict__ table,
                                  long long ldt, const long long* __restrict__ tokens, int col0,
@@ -138,6 +211,27 @@ hipError_t sm_group_rms(int dt_in, int dt_out, const void* x, long long ldx, con
   }
   SM_DISPATCH(dt_out, CALL_O)
 #undef CALL_O
+  return hipGetLastError();
+}
+
+// x fp32 [rows][W] contiguous; g [rows][W] with row stride ldg; w fp32 [W], or [W / groups] with
+// shared_w; out [rows][W] contiguous.  W * 4 bytes of LDS.
+hipError_t sm_gated_rms(int dt, const float* x, const void* g, long long ldg, const float* w,
+                        void* out, int rows, int W, int groups, int shared_w, int gate_first,
+                        int sigmoid, float eps, hipStream_t st) {
+  if (rows == 0) return hipSuccess;
+  if (groups < 1 || W < 1 || W % groups || (size_t)W * sizeof(float) > 65536 - 64)
+    return hipErrorInvalidValue;
+  const bool vec = (W / groups) % 4 == 0 && ldg % 4 == 0 && (uintptr_t)x % 16 == 0 &&
+                   (uintptr_t)g % 16 == 0 && (uintptr_t)out % 16 == 0;
+  const size_t lds = (size_t)W * sizeof(float);
+#define CALL(TT)                                                                                \
+  if (vec) gated_rms_kernel<TT, true><<<rows, 256, lds, st>>>(x, (const TT*)g, ldg, w, (TT*)out, \
+                                                W, groups, shared_w, gate_first, sigmoid, eps); \
+  else gated_rms_kernel<TT, false><<<rows, 256, lds, st>>>(x, (const TT*)g, ldg, w, (TT*)out, W, \
+                                                groups, shared_w, gate_first, sigmoid, eps)
+  SM_DISPATCH(dt, CALL)
+#undef CALL
   return hipGetLastError();
 }
 

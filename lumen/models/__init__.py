@@ -1,7 +1,8 @@
 """Model families: Llama / Llama-2 (7B, 13B, 70B-GQA), OPT (125m), Gedatar (hybrid stack),
 Dalavik (latent + grouped-query attention stack), Fanopel (gated window attention + routed
-experts) and Foderax (parallel sigmoid-attention / minGRU, latent and differential attention
-layers with routed experts and depth-weighted layer inputs)."""
+experts), Foderax (parallel sigmoid-attention / minGRU, latent and differential attention
+layers with routed experts and depth-weighted layer inputs) and Silonex (window attention beside
+a gated delta rule, lightning attention, state-space duality; hyper-connections, looped layers)."""
 from __future__ import annotations
 
 from typing import Optional
@@ -15,11 +16,12 @@ from .foderax import FoderaxForCausalLM  # noqa: F401
 from .gedatar import GedatarForCausalLM  # noqa: F401
 from .llama import LlamaForCausalLM  # noqa: F401
 from .opt import OPTForCausalLM  # noqa: F401
+from .silonex import SilonexForCausalLM  # noqa: F401
 
 
 MODEL_CLASSES = {"llama": LlamaForCausalLM, "opt": OPTForCausalLM, "gedatar": GedatarForCausalLM,
                  "dalavik": DalavikForCausalLM, "fanopel": FanopelForCausalLM,
-                 "foderax": FoderaxForCausalLM}
+                 "foderax": FoderaxForCausalLM, "silonex": SilonexForCausalLM}
 
 
 def build_model(name_or_cfg, dtype=torch.bfloat16, device=None, init: str = "auto",

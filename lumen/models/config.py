@@ -17,7 +17,7 @@ from typing import Optional
 
 @dataclass
 class ModelConfig:
-    arch: str = "llama"  # "llama" | "opt" | "gedatar" | "dalavik" | "fanopel" | "foderax"
+    arch: str = "llama"  # "llama" | "opt" | "gedatar" | "dalavik" | "fanopel" | "foderax" | "silonex"
     vocab_size: int = 32000
     hidden_size: int = 4096
     intermediate_size: int = 11008
@@ -55,12 +55,18 @@ class ModelConfig:
     # ``embedding_scale``; logits pass through cap * tanh(. / cap) when ``logit_softcap`` > 0
     embedding_scale: float = 1.0
     logit_softcap: float = 0.0
+    # Silonex (layer_specs of "parallel" | "lightning" | "mamba2" mixers): copies of the residual
+    # stream, the layers that run several times in a row ({"start", "stop", "times"} or None) and
+    # the factor of the logits
+    streams: int = 1
+    loop: Optional[dict] = None
+    logit_scale: float = 1.0
 
     @property
     def is_hybrid(self) -> bool:
         """Every layer names its own mixer and keeps its own kind of cache or state; such a stack
         is served by ``serve.hybrid_runner`` on the step's row segments."""
-        return self.arch in ("gedatar", "dalavik", "fanopel", "foderax")
+        return self.arch in ("gedatar", "dalavik", "fanopel", "foderax", "silonex")
 
     @property
     def head_dim(self) -> int:
@@ -84,6 +90,8 @@ class ModelConfig:
                 from .fanopel import tensor_shapes
             elif self.arch == "foderax":
                 from .foderax import tensor_shapes
+            elif self.arch == "silonex":
+                from .silonex import tensor_shapes
             else:
                 from .dalavik import tensor_shapes
 
@@ -240,7 +248,44 @@ def foderax_to_dict(cfg: ModelConfig) -> dict:
             "eos_token_id": cfg.eos_token_id}
 
 
+def _silonex_to_config(d: dict) -> ModelConfig:
+    """config.json of a Silonex checkpoint: {"architecture": "Silonex", "vocab", "width",
+    "streams", "loop": {"start", "stop", "times"}, "logit_scale", "norm": {"eps"}, "layers":
+    [{"type", "mixer", "mlp"}, ...]}."""
+    layers = d["layers"]
+    if not layers:
+        raise ValueError("a Silonex config needs at least one layer")
+    for i, L in enumerate(layers):
+        if L.get("type") not in ("parallel", "lightning", "mamba2"):
+            raise ValueError(f"layer {i}: unknown mixer type {L.get('type')!r}")
+        kind = (L.get("mlp") or {}).get("kind", "dense")
+        if kind != "dense":
+            raise ValueError(f"layer {i}: unknown feed-forward kind {kind!r}")
+    return ModelConfig(
+        arch="silonex", vocab_size=int(d["vocab"]), hidden_size=int(d["width"]),
+        num_hidden_layers=len(layers), rms_norm_eps=float(d["norm"]["eps"]),
+        streams=int(d.get("streams", 1)), loop=d.get("loop") or None,
+        logit_scale=float(d.get("logit_scale", 1.0)), layer_specs=layers, intermediate_size=0,
+        num_attention_heads=0, num_key_value_heads=0, max_position_embeddings=1 << 20,
+        tie_word_embeddings=True, bos_token_id=int(d.get("bos_token_id", 0)),
+        eos_token_id=int(d.get("eos_token_id", -1)), pad_token_id=int(d.get("pad_token_id", 0)),
+        name=d.get("_name_or_path", "silonex"))
+
+
+def silonex_to_dict(cfg: ModelConfig) -> dict:
+    """The checkpoint form of a Silonex configuration (inverse of ``_silonex_to_config``)."""
+    d = {"architecture": "Silonex", "vocab": cfg.vocab_size, "width": cfg.hidden_size,
+         "streams": cfg.streams, "logit_scale": cfg.logit_scale,
+         "norm": {"eps": cfg.rms_norm_eps}, "layers": cfg.layer_specs,
+         "eos_token_id": cfg.eos_token_id}
+    if cfg.loop:
+        d["loop"] = cfg.loop
+    return d
+
+
 def _hf_to_config(d: dict) -> ModelConfig:
+    if d.get("architecture") == "Silonex":
+        return _silonex_to_config(d)
     if d.get("architecture") == "Foderax":
         return _foderax_to_config(d)
     if d.get("architecture") == "Fanopel":
@@ -415,6 +460,30 @@ PRESETS = {
                                             "rot": {"base": 5000.0, "dims": 8}},
              "mlp": {"kind": "moe", "expert": {"ff": 40},
                      "router": {"experts": 6, "top": 3, "groups": {"count": 3, "keep": 2}}}}]),
+    # residual stream in three copies; a looped pair of layers (window attention beside a gated
+    # delta rule, state-space duality), lightning attention, one layer without a feed-forward
+    "tiny-silonex": dict(
+        arch="silonex", vocab_size=336, hidden_size=96, num_hidden_layers=4, rms_norm_eps=1e-5,
+        streams=3, loop={"start": 1, "stop": 3, "times": 2}, logit_scale=1.5, intermediate_size=0,
+        num_attention_heads=0, num_key_value_heads=0, max_position_embeddings=1 << 20,
+        eos_token_id=-1, tie_word_embeddings=True, name="tiny-silonex", layer_specs=[
+            {"type": "lightning", "mixer": {"heads": 3, "dim": 24, "vdim": 16,
+                                            "decay": [0.5, 0.9, 0.99]},
+             "mlp": {"kind": "dense", "ff": 160}},
+            {"type": "parallel", "mixer": {
+                "left": {"heads": 4, "kv_heads": 2, "dim": 32, "vdim": 24, "scale": 0.2,
+                         "softcap": 15.0, "mask": {"size": 40},
+                         "rot": {"base": 5000.0, "dims": 16,
+                                 "scaling": {"factor": 4.0, "low": 1.0, "high": 4.0,
+                                             "original": 256}}},
+                "right": {"heads": 4, "kv_heads": 2, "dim": 16, "vdim": 24, "conv": 4}},
+             "mlp": {"kind": "dense", "ff": 128}},
+            {"type": "mamba2", "mixer": {"heads": 6, "vdim": 16, "state": 24, "groups": 2,
+                                         "norm_groups": 3, "conv": 4},
+             "mlp": None},
+            {"type": "mamba2", "mixer": {"heads": 4, "vdim": 32, "state": 16, "groups": 1,
+                                         "norm_groups": 1, "conv": 2},
+             "mlp": {"kind": "dense", "ff": 96}}]),
     "tiny-opt": dict(arch="opt", vocab_size=512, hidden_size=64, intermediate_size=256,
                      ffn_dim=256, num_hidden_layers=2, num_attention_heads=4,
                      num_key_value_heads=4, max_position_embeddings=256, word_embed_proj_dim=64,

@@ -43,7 +43,7 @@ SIGNATURES = {
                    "pi" "ipp",
     "sm_win_attn_tiles": "iplppppl" "pi" "pi" "pp" "iiii" "ff" "p" "iii" "ipi",
     "sm_row_norm_write": "iplpppppiiif",
-    "sm_layer_norm": "iippfppiif",
+    "sm_layer_norm": "iippfpppiif",
     "sm_embed_pos": "ipppppiiii",
     "sm_route_groups": "pppiiiiiiffii",
     "sm_rotary_write": "iplppppiiiiipii",
@@ -53,6 +53,13 @@ SIGNATURES = {
     "sm_embed_scaled": "ipppiiif",
     "sm_soft_cap": "ipplf",
     "sm_scaled_act": "ipppiiiii",
+    "sm_gated_rms": "ipplppiiiiiif",
+    "sm_hyper_mix": "i" "pppi" "ppppf" "ppp" "ppf" "pp" "iiii",
+    "sm_head_norm_rotary": "ipl" "ppppppp" "iiiiiiif",
+    "sm_head_scan_chunk": "ii" "plplplplpl" "pppp" "pp" "ppp" "iiiiiiff",
+    "sm_head_scan_step": "ii" "plplplplpl" "pppp" "pp" "ppp" "iiiiiiff",
+    "sm_short_conv": "iplpppp" "pppp" "iii",
+    "sm_conv_tail": "iiplpppp" "ppp" "iii",
 }
 
 

@@ -675,6 +675,62 @@ def head_norm_write(qkv: torch.Tensor, wq: torch.Tensor, wk: torch.Tensor, slots
          qkv.shape[0], H, G, D, Dv, eps)
 
 
+def head_norm_rotary_write_ref(z, wq, wk, positions, slots, kcache, vcache, H, G, D, Dv, dims,
+                               inv_freq, eps, value_norm):
+    T = z.shape[0]
+
+    def unit(x):
+        return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
+
+    def turn(x):
+        if not dims:
+            return x
+        a = positions.float().view(T, 1, 1) * inv_freq.float().view(1, 1, -1)
+        c, s = torch.cos(a), torch.sin(a)
+        u, v = x[..., :dims // 2], x[..., dims // 2:dims]
+        return torch.cat([u * c - v * s, v * c + u * s, x[..., dims:]], -1)
+
+    q = turn(unit(z[:, :H * D].float().reshape(T, H, D)) * wq.float())
+    k = turn(unit(z[:, H * D:(H + G) * D].float().reshape(T, G, D)) * wk.float())
+    v = z[:, (H + G) * D:(H + G) * D + G * Dv].float().reshape(T, G, Dv)
+    v = unit(v) if value_norm else v
+    z[:, :H * D] = q.reshape(T, H * D).to(z.dtype)
+    ok = slots >= 0
+    kcache.view(-1, G, D)[slots[ok]] = k[ok].to(kcache.dtype)
+    vcache.view(-1, G, Dv)[slots[ok]] = v[ok].to(vcache.dtype)
+
+
+def head_norm_rotary_write(z: torch.Tensor, wq: torch.Tensor, wk: torch.Tensor,
+                           positions: torch.Tensor, slots: torch.Tensor, kcache: torch.Tensor,
+                           vcache: torch.Tensor, H: int, G: int, D: int, Dv: int, dims: int,
+                           inv_freq: torch.Tensor, eps: float, value_norm: bool = False) -> None:
+    """z [T, >= (H + G) * D + G * Dv] (a fused projection's output; further columns are left
+    alone): every query and key head is RMS-normed over its D entries with the weight ``wq`` /
+    ``wk`` [D] shared by the heads, then turned on its first ``dims`` entries in the half layout
+    by position * ``inv_freq``; with ``value_norm`` every value head is divided by its own root mean
+    square.  q is replaced in place, k and v go to their paged caches at ``slots`` (int64; -1
+    skips).  Norms, angles and rotation are fp32.  (HIP: ``csrc/seqmix/hyper.hip``.)"""
+    from ._seqmix import DT, call, use_seqmix
+
+    if dims % 2 or dims > D:
+        raise ValueError(f"rotary dims {dims} must be even and at most the head size {D}")
+    if z.shape[1] < (H + G) * D + G * Dv:
+        raise ValueError(f"z has {z.shape[1]} columns, expected at least {(H + G) * D + G * Dv}")
+    if tuple(kcache.shape[2:]) != (G, D) or tuple(vcache.shape[2:]) != (G, Dv):
+        raise ValueError(f"caches {tuple(kcache.shape)} / {tuple(vcache.shape)} do not hold {G} "
+                         f"heads of {D} / {Dv}")
+    if not use_seqmix(z):
+        return head_norm_rotary_write_ref(z, wq, wk, positions, slots, kcache, vcache, H, G, D, Dv,
+                                          dims, inv_freq, eps, value_norm)
+    assert z.stride(1) == 1 and kcache.is_contiguous() and vcache.is_contiguous()
+    assert kcache.dtype == z.dtype and vcache.dtype == z.dtype and positions.dtype == torch.int32
+    assert wq.dtype == torch.float32 and wk.dtype == torch.float32
+    assert wq.numel() == D and wk.numel() == D
+    assert inv_freq.dtype == torch.float32 and inv_freq.numel() >= dims // 2
+    call("sm_head_norm_rotary", DT[z.dtype], z, z.stride(0), wq, wk, positions, slots, kcache,
+         vcache, inv_freq, z.shape[0], H, G, D, Dv, dims, int(bool(value_norm)), eps)
+
+
 def row_norm_write_ref(qk, wq, wk, slots, kcache, vcache, HD, GD, eps):
     def unit(x):
         x = x.float()
@@ -924,7 +980,7 @@ def row_attention(q1: torch.Tensor, q2: Optional[torch.Tensor], kcache: torch.Te
 # query head within the key head).  Head h = g * rep + r becomes
 #     o = a[g, 0, r] - lam * a[g, 1, r];   o <- o / sqrt(mean(o^2) + eps) * out_scale
 # and the concatenated heads are multiplied element-wise by sigmoid(gate).  fp32 throughout; only
-# the stored result is rounded.  (HIP: ``csrc/seqmix/foderax.hip``.)
+# the stored result is rounded.  (HIP: ``csrc/seqmix/depth_mix.hip``.)
 def diff_head_combine_ref(a, lam, out_scale, eps, gate, G, rep, Dv):
     T = a.shape[0]
     af = a.float().reshape(T, G, 2, rep, Dv)

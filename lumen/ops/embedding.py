@@ -80,7 +80,7 @@ def embed_scaled(tokens: torch.Tensor, table: torch.Tensor, scale: float,
                  out: torch.Tensor) -> torch.Tensor:
     """table[token] * scale per row in fp32 into ``out`` [T, W] (fp32, contiguous): the start of a
     residual stream whose embedding is multiplied by a constant.  (HIP
-    ``csrc/seqmix/foderax.hip``.)"""
+    ``csrc/seqmix/depth_mix.hip``.)"""
     from ._seqmix import DT, call, use_seqmix
 
     if not use_seqmix(table):

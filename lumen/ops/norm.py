@@ -184,48 +184,162 @@ def group_rms_residual(x: torch.Tensor, y: torch.Tensor, w: torch.Tensor, groups
     return x, xb
 
 
-# ---- layer norm with a weight and no shift, fused with a scaled residual add -------------------
-# LN(x) = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w.  The fp32 residual stream takes a
+# ---- layer norm with a weight (and optionally a shift), fused with a scaled residual add ----------
+# LN(x) = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w (+ b).  The fp32 residual stream takes a
 # sublayer's output multiplied by a constant, x += mult * y, and the same pass produces the next
 # sublayer's input LN(x) in the model dtype.  fp32 throughout; only a stored result is rounded.
 # (HIP: ``csrc/seqmix/layer_norm.hip``.)
-def weight_layer_norm_ref(x, w, eps, out_dtype=None):
+def weight_layer_norm_ref(x, w, eps, out_dtype=None, b=None):
     xf = x.float()
     d = xf - xf.mean(-1, keepdim=True)
     y = d / torch.sqrt((d * d).mean(-1, keepdim=True) + eps) * w.float()
+    if b is not None:
+        y = y + b.float()
     return y.to(out_dtype or x.dtype)
 
 
-def scaled_residual_layer_norm_ref(x, y, mult, w, eps, out_dtype=None):
+def scaled_residual_layer_norm_ref(x, y, mult, w, eps, out_dtype=None, b=None):
     if y is not None:
         x.add_(y.float(), alpha=mult)
-    return x, (weight_layer_norm_ref(x, w, eps, out_dtype or x.dtype) if w is not None else None)
+    return x, (weight_layer_norm_ref(x, w, eps, out_dtype or x.dtype, b) if w is not None
+               else None)
 
 
 def scaled_residual_layer_norm(x: torch.Tensor, y: Optional[torch.Tensor], mult: float,
-                               w: Optional[torch.Tensor], eps: float, out_dtype=None):
+                               w: Optional[torch.Tensor], eps: float, out_dtype=None,
+                               b: Optional[torch.Tensor] = None):
     """The fp32 residual stream ``x`` [T, W] takes ``mult * y`` in place (``y`` None: nothing is
-    added) and -- fused, when ``w`` [W] (fp32) is given -- h = LN(x) * w is produced in
+    added) and -- fused, when ``w`` [W] (fp32) is given -- h = LN(x) * w (+ ``b``) is produced in
     ``out_dtype``.  Returns (x, h or None)."""
     from ._seqmix import DT, call, use_seqmix
 
     if not use_seqmix(x):
-        return scaled_residual_layer_norm_ref(x, y, mult, w, eps, out_dtype)
+        return scaled_residual_layer_norm_ref(x, y, mult, w, eps, out_dtype, b)
     assert x.dtype == torch.float32 and x.is_contiguous()
     assert y is None or (y.is_contiguous() and y.shape == x.shape)
     assert w is None or (w.dtype == torch.float32 and w.is_contiguous())
+    assert b is None or (b.dtype == torch.float32 and b.is_contiguous())
     if y is None and w is None:
         return x, None
     out_dtype = out_dtype or (y.dtype if y is not None else x.dtype)
     h = torch.empty(x.shape, dtype=out_dtype, device=x.device) if w is not None else None
     call("sm_layer_norm", DT[y.dtype] if y is not None else 0, DT[out_dtype], x, y, float(mult), w,
-         h, x.shape[0], x.shape[1], eps)
+         b, h, x.shape[0], x.shape[1], eps)
     return x, h
 
 
-def weight_layer_norm(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype=None) -> torch.Tensor:
-    """LN(x) * w of the fp32 rows ``x`` [T, W] in ``out_dtype``."""
-    return scaled_residual_layer_norm(x, None, 0.0, w, eps, out_dtype or x.dtype)[1]
+def weight_layer_norm(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype=None,
+                      b: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """LN(x) * w (+ ``b``) of the fp32 rows ``x`` [T, W] in ``out_dtype``."""
+    return scaled_residual_layer_norm(x, None, 0.0, w, eps, out_dtype or x.dtype, b)[1]
+
+
+# ---- a recurrence's read-out: group RMS norm and output gate ---------------------------------------
+# The fp32 row x is normed in ``groups`` equal parts (each by its own root mean square), weighted,
+# and gated by act(g) with act = SiLU or the sigmoid; the gate multiplies either before the norm or
+# after it.  fp32 throughout; only the result is rounded.  (HIP: ``csrc/seqmix/rms_group.hip``.)
+GATES = {"silu": 0, "sigmoid": 1}
+
+
+def gated_rms_norm_ref(x, g, w, groups, eps, gate, gate_first):
+    a = torch.sigmoid(g.float())
+    a = a * g.float() if gate == "silu" else a
+    xf = x.float() * a if gate_first else x.float()
+    T, W = x.shape
+    p = xf.reshape(T, groups, W // groups)
+    p = p / torch.sqrt((p * p).mean(-1, keepdim=True) + eps)
+    wf = w.float()
+    y = p.reshape(T, W) * (wf if wf.numel() == W else wf.repeat(groups))
+    return (y if gate_first else y * a).to(g.dtype)
+
+
+def gated_rms_norm(x: torch.Tensor, g: torch.Tensor, w: torch.Tensor, groups: int, eps: float,
+                   gate: str, gate_first: bool) -> torch.Tensor:
+    """``x`` [T, W] fp32 and its gate logits ``g`` [T, W] (a column slice of a fused projection is
+    fine) -> [T, W] in g's dtype; ``w`` fp32 [W], or [W / groups] shared by the groups; ``gate``:
+    silu | sigmoid; ``gate_first``: norm(x * act(g)) * w instead of norm(x) * w * act(g)."""
+    from ._seqmix import DT, call, use_seqmix
+
+    T, W = x.shape
+    if W % groups:
+        raise ValueError(f"width {W} is not a multiple of {groups} groups")
+    if w.numel() not in (W, W // groups):
+        raise ValueError(f"{w.numel()} weights for rows of {W} in {groups} groups")
+    if not use_seqmix(x):
+        return gated_rms_norm_ref(x, g, w, groups, eps, gate, gate_first)
+    assert x.dtype == torch.float32 and x.is_contiguous() and w.dtype == torch.float32
+    assert g.stride(1) == 1 and tuple(g.shape) == (T, W)
+    out = torch.empty(T, W, dtype=g.dtype, device=x.device)
+    call("sm_gated_rms", DT[g.dtype], x, g, g.stride(0), w, out, T, W, groups,
+         int(w.numel() != W), int(bool(gate_first)), GATES[gate], eps)
+    return out
+
+
+# ---- hyper-connections: a residual stream kept as several copies --------------------------------------
+# Between two sublayers, on the copies x_1 .. x_S of a row:
+#     x'_t = sum_s mix[s, t] x_s + out[t] y          (y: the sublayer's output)
+#     h    = LN(sum_t in[t] x'_t) * w + b            (the next sublayer's input)
+# fp32 throughout; only h is rounded.  (HIP: ``csrc/seqmix/hyper.hip``.)
+def hyper_start(tokens: torch.Tensor, table: torch.Tensor, S: int, w_in: torch.Tensor,
+                norm, eps: float, out_dtype):
+    """The start of a step: ``S`` copies of each token's embedding row -> (x [T, S, W] fp32,
+    h [T, W] = LN(sum_t w_in[t] x_t) * norm[0] + norm[1] in ``out_dtype``)."""
+    from ._seqmix import DT, call, use_seqmix
+
+    T, W = tokens.shape[0], table.shape[1]
+    if not use_seqmix(table):
+        x = table[tokens].float().view(T, 1, W).repeat(1, S, 1)
+        u = (x * w_in.float().view(1, S, 1)).sum(1)
+        return x, weight_layer_norm_ref(u, norm[0], eps, out_dtype, norm[1])
+    assert table.is_contiguous() and tokens.dtype == torch.int64 and tokens.is_contiguous()
+    assert table.dtype == out_dtype
+    x = torch.empty(T, S, W, dtype=torch.float32, device=table.device)
+    h = torch.empty(T, W, dtype=out_dtype, device=table.device)
+    call("sm_hyper_mix", DT[out_dtype], x, table, tokens, table.shape[0], None, None, None, None,
+         0.0, None, None, w_in, norm[0], norm[1], eps, h, None, 1, T, S, W)
+    return x, h
+
+
+def hyper_mix_ref(x, ys, pair, mix, out, w_in, norm, eps, out_dtype):
+    y = ys[0].float()
+    if len(ys) == 2:
+        wa, wb, eps_y = pair
+        rms = lambda t: t / torch.sqrt((t * t).mean(-1, keepdim=True) + eps_y)  # noqa: E731
+        y = rms(y) * wa.float() + rms(ys[1].float()) * wb.float()
+    new = torch.einsum("nsw,st->ntw", x, mix.float()) + out.float().view(1, -1, 1) * y[:, None]
+    x.copy_(new)
+    u = (x * w_in.float().view(1, -1, 1)).sum(1)
+    return u if norm is None else weight_layer_norm_ref(u, norm[0], eps, out_dtype, norm[1])
+
+
+def hyper_mix(x: torch.Tensor, ys, pair, mix: torch.Tensor, out: torch.Tensor,
+              w_in: torch.Tensor, norm, eps: float, out_dtype=None, keep: bool = True):
+    """``x`` [T, S, W] fp32 takes a sublayer's output through ``mix`` [S, S] (from, to) and ``out``
+    [S] in place (``keep`` False: the copies are not needed any more and need not be stored);
+    returns LN(sum_t w_in[t] x_t) with ``norm`` = (w, b) in ``out_dtype``, or with ``norm`` None the
+    fp32 sum itself.  ``ys``: one output [T, W] in the compute dtype, or two that are RMS-normed over
+    the row with the weights of ``pair`` = (w_a, w_b, eps) and added."""
+    from ._seqmix import DT, call, use_seqmix
+
+    T, S, W = x.shape
+    if len(ys) not in (1, 2) or (len(ys) == 2) != (pair is not None):
+        raise ValueError("one sublayer output, or two with their norms' weights")
+    out_dtype = out_dtype or ys[0].dtype
+    if not use_seqmix(x):
+        return hyper_mix_ref(x, ys, pair, mix, out, w_in, norm, eps, out_dtype)
+    if S > 8:
+        raise ValueError(f"{S} residual copies > 8 are not supported")
+    assert x.dtype == torch.float32 and x.is_contiguous()
+    for y in ys:
+        assert y.is_contiguous() and tuple(y.shape) == (T, W) and y.dtype == out_dtype
+    for f in (mix, out, w_in) + tuple(norm or ()) + tuple((pair or ())[:2]):
+        assert f.dtype == torch.float32 and f.is_contiguous()
+    dst = torch.empty(T, W, dtype=torch.float32 if norm is None else out_dtype, device=x.device)
+    wa, wb, eps_y = pair if pair is not None else (None, None, 0.0)
+    call("sm_hyper_mix", DT[out_dtype], x, None, None, 0, ys[0], ys[1] if len(ys) == 2 else None,
+         wa, wb, eps_y, mix, out, w_in, norm[0] if norm else None, norm[1] if norm else None, eps,
+         dst if norm else None, None if norm else dst, int(bool(keep)), T, S, W)
+    return dst
 
 
 # ---- depth-weighted layer inputs: layer scale, history, weighted average, next norm ---------------
@@ -234,7 +348,7 @@ def weight_layer_norm(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype=No
 #     X_n = x + sum_k scale_k * y_k          (the sublayers' outputs with per-channel scales)
 #     x  <- sum_{j <= n} mix[j] * X_j         (what the next layer reads)
 #     h   = x / sqrt(mean(x^2) + eps) * w     (its norm, in the compute dtype)
-# fp32 throughout; only h is rounded.  (HIP: ``csrc/seqmix/foderax.hip``.)
+# fp32 throughout; only h is rounded.  (HIP: ``csrc/seqmix/depth_mix.hip``.)
 def depth_mix_norm_ref(hist, n, x, ys, scales, mix, w, eps, out_dtype):
     new = x.float().clone()
     for y, sc in zip(ys, scales):

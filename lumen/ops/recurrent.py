@@ -204,3 +204,97 @@ def min_gru_scan(zxg: torch.Tensor, b_z: torch.Tensor, b_x: torch.Tensor, state:
         call("sm_min_gru", DT[zxg.dtype], zxg, zxg.stride(0), b_z, b_x, state, out, seg.cu[P:],
              seg.slot[P:], seg.start[P:], seg.S - P, width, float(shift), None, None, 0, 0)
     return out
+
+
+# ---- matrix state with ONE decay per (token, head): linear attention, state-space duality, delta ----
+# ``head_scan`` runs, per head, with S [Dk, Dv] fp32 from zero at a sequence's first token:
+#   linear   S <- e^l S + k (dt v)^T;                                     o = S^T q (+ skip v)
+#   delta    S <- e^l S;  u = beta (v - S^T k);  S <- S + k u^T;          o = S^T q
+# l is a constant per head (``log_decay``; dt = 1) or per token: dt = softplus(a + dt_bias),
+# l = -exp(A_log) dt (the delta rule uses dt in the decay only).  The delta rule first makes q and k
+# unit vectors, x / sqrt(sum x^2 + key_eps), and multiplies q by ``q_scale``.  Decays, step sizes,
+# unit vectors and the state are fp32; the read-out is returned in fp32.
+# (HIP: ``csrc/seqmix/head_scan_chunk.hip`` for prompt portions, ``head_scan_step.hip`` for decoded
+# rows.)
+def head_scan_ref(q, k, v, state, seg: SegBatch, H, rep, Dk, Dv, decay, beta=None, skip=None,
+                  silu_in=False, key_eps=0.0, q_scale=1.0):
+    T = q.shape[0]
+    act = F.silu if silu_in else (lambda t: t)
+    hg = torch.arange(H, device=q.device) // rep
+    q_ = act(q.float().reshape(T, H // rep, Dk))
+    k_ = act(k.float().reshape(T, H // rep, Dk))
+    v_ = act(v.float().reshape(T, H, Dv))
+    if beta is not None:
+        q_ = q_ / torch.sqrt((q_ * q_).sum(-1, keepdim=True) + key_eps) * q_scale
+        k_ = k_ / torch.sqrt((k_ * k_).sum(-1, keepdim=True) + key_eps)
+        b_ = torch.sigmoid(beta.float())
+    q_, k_ = q_[:, hg], k_[:, hg]
+    if isinstance(decay, torch.Tensor):
+        g = torch.exp(decay.float()).view(1, H).expand(T, H)
+        dt = torch.ones(T, H, device=q.device)
+    else:
+        a, A_log, dt_bias = decay
+        dt = F.softplus(a.float() + dt_bias.float())
+        g = torch.exp(-torch.exp(A_log.float()) * dt)
+    out = torch.empty(T, H, Dv, dtype=torch.float32, device=q.device)
+    cu, slots, starts = seg.cu.tolist(), seg.slot.tolist(), seg.start.tolist()
+    for s in range(seg.S):
+        i0, i1 = cu[s], cu[s + 1]
+        if i1 == i0:
+            continue
+        S = state[slots[s]].clone() if starts[s] > 0 else torch.zeros_like(state[slots[s]])
+        for t in range(i0, i1):
+            S = g[t].view(H, 1, 1) * S
+            if beta is not None:
+                u = b_[t].view(H, 1) * (v_[t] - torch.einsum("hkv,hk->hv", S, k_[t]))
+            else:
+                u = dt[t].view(H, 1) * v_[t]
+            S = S + k_[t][:, :, None] * u[:, None, :]
+            out[t] = torch.einsum("hkv,hk->hv", S, q_[t])
+        state[slots[s]] = S
+    if skip is not None:
+        out = out + skip.float().view(1, H, 1) * v_
+    return out.reshape(T, H * Dv)
+
+
+def head_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor,
+              seg: SegBatch, H: int, Dk: int, Dv: int, decay, beta=None, skip=None, rep: int = 1,
+              silu_in: bool = False, key_eps: float = 0.0, q_scale: float = 1.0) -> torch.Tensor:
+    """q, k [T, (H / rep) * Dk] (head h reads block h // rep), v [T, H * Dv]: rows with a unit column
+    stride (slices of wider buffers are fine); ``state`` [slots, H, Dk, Dv] fp32 moves on.  ``decay``:
+    an fp32 tensor [H] of constant log decays, or (logits [T, H], A_log [H], dt_bias [H]).  ``beta``
+    [T, H] (write-strength logits) selects the delta rule, without ``skip``.  ``silu_in``: q, k and v
+    pass through silu as they are read.  Returns the read-outs [T, H * Dv] in fp32."""
+    from ._seqmix import DT, call, use_seqmix
+
+    if H % rep:
+        raise ValueError(f"{H} heads do not share q / k in groups of {rep}")
+    const = isinstance(decay, torch.Tensor)
+    if beta is not None and (const or skip is not None):
+        raise ValueError("the delta rule takes per-token decays and no skip")
+    if not use_seqmix(q):
+        return head_scan_ref(q, k, v, state, seg, H, rep, Dk, Dv, decay, beta, skip, silu_in,
+                             key_eps, q_scale)
+    if Dk > 256:
+        raise ValueError(f"recurrent key size {Dk} > 256 is not supported")
+    assert state.dtype == torch.float32 and state.is_contiguous()
+    assert tuple(state.shape[1:]) == (H, Dk, Dv)
+    assert q.shape[1] == k.shape[1] == H // rep * Dk and v.shape[1] == H * Dv
+    assert q.dtype == k.dtype == v.dtype
+    al, A_log, dt_bias = (None, None, None) if const else decay
+    for f in (decay if const else A_log, dt_bias, skip):
+        assert f is None or (f.dtype == torch.float32 and f.is_contiguous() and f.numel() == H)
+    for f in (al, beta):
+        assert f is None or (tuple(f.shape) == (q.shape[0], H) and f.dtype == q.dtype)
+    T = q.shape[0]
+    out = torch.empty(T, H * Dv, dtype=torch.float32, device=q.device)
+    head = (DT[q.dtype], int(beta is not None), q, _ld(q), k, _ld(k), v, _ld(v), al,
+            _ld(al) if al is not None else 0, beta, _ld(beta) if beta is not None else 0, A_log,
+            dt_bias, decay if const else None, skip, state, out)
+    tail = (H, rep, Dk, Dv, int(bool(silu_in)), key_eps, q_scale)
+    P, _ = seg.portions()
+    if P:
+        call("sm_head_scan_chunk", *head, seg.cu, seg.slot, seg.start, P, *tail)
+    if seg.S > P:
+        call("sm_head_scan_step", *head, seg.cu[P:], seg.slot[P:], seg.start[P:], seg.S - P, *tail)
+    return out

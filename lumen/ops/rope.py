@@ -7,6 +7,7 @@ the token-major QKV buffer at arbitrary positions.
 """
 from __future__ import annotations
 
+import math
 from typing import Dict, Optional, Tuple
 
 import torch
@@ -171,6 +172,32 @@ def interleaved_inv_freq(dims: int, base: float, device) -> torch.Tensor:
     if t is None:
         t = torch.tensor([float(base) ** (-2.0 * i / dims) for i in range(dims // 2)],
                          dtype=torch.float64).float().to(device)
+        _INV_FREQ[key] = t
+    return t
+
+
+def stretched_inv_freq(dims: int, base: float, scaling, device) -> torch.Tensor:
+    """[dims / 2] fp32 rotations per position, base^(-2i / dims), stretched by wavelength when
+    ``scaling`` = {factor, low, high, original} is given: with l = 2 pi / f, f is kept where
+    l < original / high, divided by ``factor`` where l > original / low, and blended between
+    (weight (original / l - low) / (high - low) on the kept one).  Computed in float64."""
+    if not scaling:
+        return interleaved_inv_freq(dims, base, device)
+    factor, low, high, orig = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
+    key = (int(dims), float(base), factor, low, high, orig, str(device))
+    t = _INV_FREQ.get(key)
+    if t is None:
+        fs = []
+        for i in range(dims // 2):
+            f = float(base) ** (-2.0 * i / dims)
+            wave = 2.0 * math.pi / f
+            if wave > orig / low:
+                f = f / factor
+            elif wave >= orig / high:
+                s = (orig / wave - low) / (high - low)
+                f = (1.0 - s) * f / factor + s * f
+            fs.append(f)
+        t = torch.tensor(fs, dtype=torch.float64).float().to(device)
         _INV_FREQ[key] = t
     return t
 

@@ -36,6 +36,14 @@ class SegBatch:
     def T(self) -> int:
         return self.row_seg.shape[0]
 
+    def portions(self) -> tuple:
+        """(segments, rows) of the step's prompt portions, which come first; the segments after
+        them are decoded rows, one row each.  A batch without a tile list is all decoded rows
+        when it has as many segments as rows, else all portions."""
+        if self.q_tiles is not None and self.tile_rows > 0:
+            return self.S - (self.T - self.tile_rows), self.tile_rows
+        return (0, 0) if self.S == self.T else (self.S, self.T)
+
 
 import os
 

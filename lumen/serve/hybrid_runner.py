@@ -1,11 +1,12 @@
 """Serving runner for stacks whose layers each name their own mixer (Gedatar, Dalavik,
-Fanopel, Foderax): paged caches + per-sequence recurrent state.
+Fanopel, Foderax, Silonex): paged caches + per-sequence recurrent state.
 
-Four families share the runner, the segments, the block manager and the hipGraph decode; each
+Five families share the runner, the segments, the block manager and the hipGraph decode; each
 has its weights class (stacked projections, fp32 constants), its caches and its step function:
 Gedatar (``HybridWeights`` / ``HybridState`` / ``run_layers``, described next), Dalavik
-(``DalavikWeights`` / ``DalavikState``), Fanopel (``FanopelWeights`` / ``FanopelState``) and
-Foderax (``FoderaxWeights`` / ``FoderaxState``), further down.
+(``DalavikWeights`` / ``DalavikState``), Fanopel (``FanopelWeights`` / ``FanopelState``),
+Foderax (``FoderaxWeights`` / ``FoderaxState``) and Silonex (``SilonexWeights`` /
+``SilonexState``), further down.
 
 One step function for prefill chunks, decode rows and mixtures of both.  The rows of a step are
 cut into segments (``ops.segments.SegBatch``: one per chunk, one per decode row); per layer
@@ -41,15 +42,16 @@ import torch.nn.functional as F
 
 from ..models.config import ModelConfig
 from ..models.gedatar import DELTA_DECAY, DELTA_KEY_EPS
-from ..ops.attention import (chunk_sink_attention, diff_head_combine, head_norm_write,
-                             latent_write, row_attention, row_norm_write, transposed_values_ok,
-                             write_key_cache)
-from ..ops.conv import dyt_canon
+from ..ops.attention import (chunk_sink_attention, diff_head_combine, head_norm_rotary_write,
+                             head_norm_write, latent_write, row_attention, row_norm_write,
+                             transposed_values_ok, write_key_cache)
+from ..ops.conv import dyt_canon, short_conv
 from ..ops.embedding import embed_positions, embed_scaled, gated_token_slice, soft_cap
 from ..ops.moe import gated_act, moe, route_groups, route_topk, router_logits
-from ..ops.norm import (depth_mix_norm, dyt, dyt_residual, group_rms_norm, group_rms_residual,
-                        scaled_residual_layer_norm, weight_layer_norm)
-from ..ops.recurrent import delta_scan, min_gru_scan, token_shift, wkv_scan
+from ..ops.norm import (depth_mix_norm, dyt, dyt_residual, gated_rms_norm, group_rms_norm,
+                        group_rms_residual, hyper_mix, hyper_start, scaled_residual_layer_norm,
+                        weight_layer_norm)
+from ..ops.recurrent import delta_scan, head_scan, min_gru_scan, token_shift, wkv_scan
 from ..ops.rope import rotary_write, rotate_interleaved_
 from ..ops.segments import SegBatch, whole_sequences
 from .model_runner import ModelRunner, StepInput
@@ -179,6 +181,15 @@ def key_bytes_per_token(cfg: ModelConfig, dtype_bytes: int = 2) -> int:
             elif m.get("kv_from") is None:
                 n += m["kv_heads"] * (2 * m["dim"] + m["vdim"])
         return max(1, n * dtype_bytes)
+    if cfg.arch == "silonex":                  # every pass of a looped layer has its own cache
+        from ..models.silonex import layer_runs
+
+        n = 0
+        for i in layer_runs(cfg):
+            if cfg.layer_specs[i]["type"] == "parallel":
+                a = cfg.layer_specs[i]["mixer"]["left"]
+                n += a["kv_heads"] * (a["dim"] + a["vdim"])
+        return max(1, n * dtype_bytes)
     if cfg.arch == "dalavik":
         n = 0
         for L in cfg.layer_specs:
@@ -192,12 +203,21 @@ def key_bytes_per_token(cfg: ModelConfig, dtype_bytes: int = 2) -> int:
                       if L["type"] == "attention") * dtype_bytes)
 
 
-def state_bytes_per_slot(cfg: ModelConfig) -> int:
+def state_bytes_per_slot(cfg: ModelConfig, dtype_bytes: int = 2) -> int:
     if cfg.arch in ("dalavik", "fanopel"):
         return 0
     if cfg.arch == "foderax":
         return 4 * sum(L["mixer"]["right"]["width"] for L in cfg.layer_specs
                        if L["type"] == "parallel")
+    if cfg.arch == "silonex":
+        from ..models.silonex import layer_runs
+
+        n = 0
+        for i in layer_runs(cfg):
+            m = cfg.layer_specs[i]["mixer"]
+            H, Dk, Dv, C, K = _silonex_state_sizes(cfg.layer_specs[i]["type"], m)
+            n += 4 * H * Dk * Dv + dtype_bytes * C * (K - 1)
+        return n
     n = 0
     for L in cfg.layer_specs:
         n += max(cfg.canon_taps - 1, 0) * cfg.hidden_size
@@ -857,8 +877,246 @@ def run_foderax_layers(w: FoderaxWeights, st: FoderaxState, tokens: torch.Tensor
     return x
 
 
+# ---- Silonex: several copies of the residual stream, looped layers, matrix-state recurrences ---------
+#
+#   x [T, S, W] fp32 = S copies of the embedding row;  h = LN(sum_s in[s] x_s)          (hyper_start)
+#   per pass of a layer (a looped layer: the same weights, its own caches and state)
+#   parallel
+#       z  = [W_q ; W_k ; W_v | W_q' ; W_k' ; W_v' | W_g ; W_b ; W_a] h     one GEMM
+#       q, k normed per head and turned, v divided by its rms; k, v to their caches
+#                                                                      (head_norm_rotary_write)
+#       o  = row_attention(soft cap, window);                y_l = W_ol o
+#       c  = silu(conv(z's q' | k' | v'))                    (short_conv, one pass over all three)
+#       r  = head_scan(delta rule);                          y_r = W_or (rms(r) w silu(g))
+#   lightning
+#       z  = [W_q ; W_k ; W_v ; W_g] h;  r = head_scan(constant decays, silu on q, k, v)
+#       y  = W_o (rms(r) w sigmoid(g))                       (gated_rms_norm)
+#   mamba2
+#       z  = W_in h;  c = silu(conv(z's x | B | C) + bias);  r = head_scan(dt-scaled, D skip)
+#       y  = W_o (grouped rms(r silu(z)) w)                  (gated_rms_norm, gate first)
+#   x <- mix, out, y;  h = LN(next in . x)                   (hyper_mix, one pass; the parallel
+#                                                            layer's two output norms and their sum too)
+#   feed-forward: [gate ; up] GEMM, silu(gate) * up, down GEMM, hyper_mix
+#   logits = (LN(sum of the copies) * logit_scale) embed^T   fp32 product of the 16-bit operands
+#
+# fp32: the copies and their sums, norms, angles, scores, softmax, decays, step sizes, beta, unit
+# vectors, states, read-outs; model dtype: GEMMs and what they store, convolution outputs.
+def _silonex_state_sizes(kind: str, m: dict) -> tuple:
+    """(heads, key size, value size, convolved channels, taps) of a mixer's recurrence."""
+    if kind == "parallel":
+        r = m["right"]
+        return (r["heads"], r["dim"], r["vdim"],
+                2 * r["kv_heads"] * r["dim"] + r["heads"] * r["vdim"], int(r["conv"]))
+    if kind == "lightning":
+        return m["heads"], m["dim"], m["vdim"], 0, 1
+    return (m["heads"], m["state"], m["vdim"],
+            m["heads"] * m["vdim"] + 2 * m["groups"] * m["state"], int(m["conv"]))
+
+
+def _stack_rows(blocks, dtype, dev):
+    """Stack blocks of projection weights row-wise, every block padded with zero rows to a multiple
+    of 8 output columns; returns (weight, the blocks' first output columns)."""
+    padded = [_pad_rows(b, dtype, dev) for b in blocks]
+    cols, n = [], 0
+    for b in padded:
+        cols.append(n)
+        n += b.shape[0]
+    return torch.cat(padded, 0).contiguous(), cols
+
+
+@dataclass
+class SilonexLayerW:
+    kind: str                       # parallel | lightning | mamba2
+    m: dict                         # the mixer's sizes and constants
+    hc: List[tuple]                 # per sublayer: (in [S], out [S], mix [S, S]) fp32
+    norms: List[tuple]              # per sublayer: (w, b) fp32
+    w: Dict[str, torch.Tensor] = field(default_factory=dict)
+    cols: List[int] = field(default_factory=list)     # first columns of the fused projection's blocks
+    ff: Optional[dict] = None       # gu [2 ff, W], down [W, ff], ff
+
+
+class SilonexWeights:
+    """Inference weights of a SilonexForCausalLM: projections that share an input are stacked into
+    one GEMM, the delta rule's three convolutions into one, the halving of a parallel layer's sum
+    is folded into its output norms' weights and the logits' factor into the final norm's; norms,
+    connection weights, decays and convolution taps are fp32.  ``runs`` lists the layer of every
+    pass: caches and state are kept per pass."""
+
+    def __init__(self, model, tp_rank: int = 0, tp_size: int = 1):
+        if tp_size != 1:
+            raise NotImplementedError("Silonex models are served at tensor-parallel size 1")
+        from ..models.silonex import UNIT_EPS, layer_runs
+        from ..ops.rope import stretched_inv_freq
+
+        cfg: ModelConfig = model.config
+        self.cfg = cfg
+        t = model.tensor
+        f32 = lambda n: t(n).detach().float().contiguous()  # noqa: E731
+        self.dtype = dt = t("embed").dtype
+        dev = t("embed").device
+        self.embed = t("embed").detach()
+        self.lm_head = self.embed                           # tied
+        scale = float(cfg.logit_scale)
+        self.final = ((f32("final.norm") * scale).contiguous(),
+                      (f32("final.norm.b") * scale).contiguous())
+        self.vocab_shard = cfg.vocab_size
+        self.runs = layer_runs(cfg)
+        self.unit_eps = float(UNIT_EPS)
+        self.ones = torch.ones(cfg.streams, dtype=torch.float32, device=dev)
+        self.layers: List[SilonexLayerW] = []
+        with torch.no_grad():
+            for i, spec in enumerate(cfg.layer_specs):
+                p, m, f = f"l{i}.", spec["mixer"], spec.get("mlp")
+                x = p + "mix."
+                subs = (1, 2) if f else (1,)
+                L = SilonexLayerW(spec["type"], m,
+                                  [tuple(f32(p + f"hc{q}.{n}") for n in ("in", "out", "mix"))
+                                   for q in subs],
+                                  [(f32(p + f"norm{q}"), f32(p + f"norm{q}.b")) for q in subs])
+                if L.kind == "parallel":
+                    a, lt, rt = m["left"], x + "left.", x + "right."
+                    L.w["in"], L.cols = _stack_rows(
+                        [[t(lt + n) for n in "qkv"], [t(rt + n) for n in "qkv"], [t(rt + "g")],
+                         [t(rt + "b")], [t(rt + "a")]], dt, dev)
+                    L.w["q.norm"], L.w["k.norm"] = f32(lt + "q.norm"), f32(lt + "k.norm")
+                    L.w["inv_freq"] = stretched_inv_freq(a["rot"]["dims"], a["rot"]["base"],
+                                                         a["rot"].get("scaling"), dev)
+                    L.w["conv"] = torch.cat([f32(rt + n + ".conv") for n in "qkv"], 0).contiguous()
+                    for n in ("A_log", "dt_bias", "norm"):
+                        L.w[n] = f32(rt + n)
+                    L.w["o_l"], L.w["o_r"] = t(lt + "o").detach(), t(rt + "o").detach()
+                    L.w["out_l"] = (0.5 * f32(lt + "out")).contiguous()
+                    L.w["out_r"] = (0.5 * f32(rt + "out")).contiguous()
+                elif L.kind == "lightning":
+                    L.w["in"], L.cols = _stack_rows([[t(x + n)] for n in "qkvg"], dt, dev)
+                    decay = torch.tensor([float(d) for d in m["decay"]], dtype=torch.float64)
+                    L.w["log_decay"] = torch.log(decay).clamp(min=-1e4).float().to(dev)
+                    L.w["norm"], L.w["o"] = f32(x + "norm"), t(x + "o").detach()
+                else:
+                    L.w["in"] = _pad_rows([t(x + "in")], dt, dev)
+                    L.w["conv"], L.w["conv.b"] = f32(x + "conv"), f32(x + "conv.b")
+                    for n in ("A_log", "dt_bias", "D", "norm"):
+                        L.w[n] = f32(x + n)
+                    L.w["o"] = t(x + "o").detach()
+                if f:
+                    y = p + "mlp."
+                    L.ff = dict(ff=int(f["ff"]), down=t(y + "down").detach(),
+                                gu=torch.cat([t(y + "gate"), t(y + "up")], 0).contiguous())
+                self.layers.append(L)
+
+    def new_state(self, slots: int, num_blocks: int, block_size: int, device):
+        return SilonexState(self, slots, num_blocks, block_size, device)
+
+    def run_layers(self, st, tokens, seg, observe=None) -> torch.Tensor:
+        return run_silonex_layers(self, st, tokens, seg, observe)
+
+    def head(self, x: torch.Tensor) -> torch.Tensor:
+        h = weight_layer_norm(x, self.final[0], self.cfg.rms_norm_eps, self.dtype, self.final[1])
+        return router_logits(h, self.lm_head)     # fp32 logits from the 16-bit (or fp32) operands
+
+
+class SilonexState:
+    """Caches and state of a Silonex model, one set per PASS of a layer (``SilonexWeights.runs``).
+    Paged through the engine's block manager: turned keys and normed values of the parallel
+    layers' attention halves.  Per state slot (+ one spare for graph padding rows): the fp32
+    matrix state [slots + 1, heads, key, value] of every recurrence and the last taps - 1 inputs of
+    its convolution [slots + 1, taps - 1, channels] in the model dtype."""
+
+    def __init__(self, w: SilonexWeights, slots: int, num_blocks: int, block_size: int, device):
+        self.slots = slots
+        self.spare = slots
+        kw = dict(dtype=w.dtype, device=device)
+        self.k: List[Optional[torch.Tensor]] = []
+        self.v: List[Optional[torch.Tensor]] = []
+        self.S: List[torch.Tensor] = []
+        self.tail: List[Optional[torch.Tensor]] = []
+        for i in w.runs:
+            L = w.layers[i]
+            H, Dk, Dv, C, K = _silonex_state_sizes(L.kind, L.m)
+            att = L.m["left"] if L.kind == "parallel" else None
+            page = (num_blocks, block_size)
+            self.k.append(torch.zeros(*page, att["kv_heads"], att["dim"], **kw) if att else None)
+            self.v.append(torch.zeros(*page, att["kv_heads"], att["vdim"], **kw) if att else None)
+            self.S.append(torch.zeros(slots + 1, H, Dk, Dv, dtype=torch.float32, device=device))
+            self.tail.append(torch.zeros(slots + 1, K - 1, C, **kw) if C else None)
+
+
+def _silonex_mixer(L: SilonexLayerW, w: SilonexWeights, st: SilonexState, n: int, h, seg) -> list:
+    """Pass ``n``'s mixer on its normed input h [T, W]: one output, or a parallel layer's two."""
+    from ..models.silonex import window
+
+    m, dt, eps = L.m, w.dtype, w.cfg.rms_norm_eps
+    T = h.shape[0]
+    z = F.linear(h, L.w["in"])
+    H, Dk, Dv, C, _ = _silonex_state_sizes(L.kind, m)
+    if L.kind == "parallel":
+        a, r = m["left"], m["right"]
+        Ha, Ga, D, Da = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+        head_norm_rotary_write(z, L.w["q.norm"], L.w["k.norm"], seg.positions, seg.cache_slots,
+                               st.k[n], st.v[n], Ha, Ga, D, Da, int(a["rot"]["dims"]),
+                               L.w["inv_freq"], eps, value_norm=True)
+        o = torch.empty(T, Ha, Da, dtype=dt, device=h.device)
+        row_attention(z[:, :Ha * D].view(T, Ha, D), None, st.k[n], st.v[n], Da, o, seg, Ha, Ga,
+                      float(a["scale"]), float(a.get("softcap") or 0.0), window=window(a))
+        _, c0, g0, b0, a0 = L.cols
+        c = short_conv(z[:, c0:c0 + C], L.w["conv"], None, st.tail[n], seg)
+        GD = r["kv_heads"] * Dk
+        y = head_scan(c[:, :GD], c[:, GD:2 * GD], c[:, 2 * GD:], st.S[n], seg, H, Dk, Dv,
+                      (z[:, a0:a0 + H], L.w["A_log"], L.w["dt_bias"]), beta=z[:, b0:b0 + H],
+                      rep=H // r["kv_heads"], key_eps=w.unit_eps, q_scale=float(Dk) ** -0.5)
+        y = gated_rms_norm(y, z[:, g0:g0 + H * Dv], L.w["norm"], H, eps, "silu", False)
+        return [F.linear(o.view(T, Ha * Da), L.w["o_l"]), F.linear(y, L.w["o_r"])]
+    if L.kind == "lightning":
+        q0, k0, v0, g0 = L.cols
+        y = head_scan(z[:, q0:q0 + H * Dk], z[:, k0:k0 + H * Dk], z[:, v0:v0 + H * Dv], st.S[n],
+                      seg, H, Dk, Dv, L.w["log_decay"], silu_in=True)
+        y = gated_rms_norm(y, z[:, g0:g0 + H * Dv], L.w["norm"], 1, eps, "sigmoid", False)
+        return [F.linear(y, L.w["o"])]
+    inner, GN = H * Dv, m["groups"] * Dk
+    c = short_conv(z[:, inner:inner + C], L.w["conv"], L.w["conv.b"], st.tail[n], seg)
+    y = head_scan(c[:, inner + GN:], c[:, inner:inner + GN], c[:, :inner], st.S[n], seg, H, Dk, Dv,
+                  (z[:, inner + C:inner + C + H], L.w["A_log"], L.w["dt_bias"]), skip=L.w["D"],
+                  rep=H // m["groups"])
+    y = gated_rms_norm(y, z[:, :inner], L.w["norm"], int(m["norm_groups"]), eps, "silu", True)
+    return [F.linear(y, L.w["o"])]
+
+
+def run_silonex_layers(w: SilonexWeights, st: SilonexState, tokens: torch.Tensor, seg: SegBatch,
+                       observe=None) -> torch.Tensor:
+    """The step function: token ids [T] + their segments -> the sum of the residual copies [T, W]
+    (fp32) after the last pass; caches and state in ``st`` move on by the step's rows.  ``observe``
+    is called with every pass's number and the sum of the copies after it."""
+    cfg = w.cfg
+    dt, eps, S = w.dtype, cfg.rms_norm_eps, cfg.streams
+    subs = [(n, q) for n, i in enumerate(w.runs) for q in range(len(w.layers[i].hc))]
+    L = w.layers[w.runs[0]]
+    x, h = hyper_start(tokens, w.embed, S, L.hc[0][0], L.norms[0], eps, dt)
+    for k, (n, q) in enumerate(subs):
+        L = w.layers[w.runs[n]]
+        pair = None
+        if q == 0:
+            ys = _silonex_mixer(L, w, st, n, h, seg)
+            if len(ys) == 2:
+                pair = (L.w["out_l"], L.w["out_r"], eps)
+        else:
+            f = L.ff
+            ys = [F.linear(gated_act(F.linear(h, f["gu"]), None, 0, 0, f["ff"]), f["down"])]
+        _, out, mix = L.hc[q]
+        last = k + 1 == len(subs)
+        if last:
+            w_in, norm = w.ones, None
+        else:
+            nn, nq = subs[k + 1]
+            nxt = w.layers[w.runs[nn]]
+            w_in, norm = nxt.hc[nq][0], nxt.norms[nq]
+        h = hyper_mix(x, ys, pair, mix, out, w_in, norm, eps, dt, keep=not last)
+        if observe is not None and q + 1 == len(L.hc):
+            observe(n, h if last else x.sum(1))
+    return h
+
+
 WEIGHTS = {"gedatar": HybridWeights, "dalavik": DalavikWeights, "fanopel": FanopelWeights,
-           "foderax": FoderaxWeights}
+           "foderax": FoderaxWeights, "silonex": SilonexWeights}
 
 
 class HybridRunner(ModelRunner):
