@@ -1,11 +1,12 @@
-"""Prefill / decode throughput of a per-layer-mixer design (Gedatar, Dalavik, Fanopel, Foderax)
-beside Llama at equal size.
+"""Prefill / decode throughput of a per-layer-mixer design (Gedatar, Dalavik, Fanopel, Foderax,
+Silonex) beside Llama at equal size.
 
-``python bench.py --hybrid [--hybrid_family dalavik|fanopel|foderax]`` (one GPU).  Fanopel also
+``python bench.py --hybrid [--hybrid_family dalavik|fanopel|foderax|silonex]`` (one GPU).  Fanopel also
 runs beside the closest design the framework already had: a Gedatar stack of attention layers
 (keys as values) with routed experts of the same shapes; Foderax beside Dalavik (latent and
-grouped-query attention through the same row kernels) and Fanopel (experts of the same shapes).
-All models get random
+grouped-query attention through the same row kernels) and Fanopel (experts of the same shapes); Silonex
+beside Gedatar (matrix-state recurrences of the same head sizes, dense feed-forwards) and Fanopel
+(window attention through the same kernels).  All models get random
 weights of layer shapes that resemble real models (width 2048 / 4096, head size 128 / 64, FFN 2.75 x width, vocab 32000), the
 same depth, and run the same forced-token workload through the serving engine
 (``lumen.serve.trace.TraceReplay``: the engine's input builder, block manager, state slots,
@@ -131,6 +132,38 @@ def foderax_config(width: int, depth_groups: int = 1):
                        name=f"foderax-w{W}", layer_specs=layers)
 
 
+def silonex_config(width: int, depth_groups: int = 1):
+    """Per group of four: a parallel layer (window attention with heads of 128, one key head per
+    four query heads, window 1024, soft cap 30, beside a gated delta rule with heads of 128, two per
+    query / key head, 4 taps), lightning attention with heads of 128, state-space duality at the
+    published shapes (inner width 2 x the model's, heads of 64, state 128, 8 groups, 4 taps), a
+    second parallel layer; dense FFN 2.75 x width; two residual copies.  No loop: a looped layer
+    only runs the same kernels again, and the depth stays comparable."""
+    from ..models.config import ModelConfig
+
+    W = width
+    H = W // 128
+    ff = {"kind": "dense", "ff": int(2.75 * W)}
+    par = {"type": "parallel", "mlp": ff, "mixer": {
+        "left": {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128,
+                 "scale": 128 ** -0.5, "softcap": 30.0, "mask": {"size": 1024},
+                 "rot": {"base": 500000.0, "dims": 128,
+                         "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}},
+        "right": {"heads": H, "kv_heads": max(1, H // 2), "dim": 128, "vdim": 128, "conv": 4}}}
+    lin = {"type": "lightning", "mlp": ff,
+           "mixer": {"heads": H, "dim": 128, "vdim": 128,
+                     "decay": [1.0 - 2.0 ** (-2 - 6 * i / H) for i in range(H)]}}
+    ssd = {"type": "mamba2", "mlp": ff,
+           "mixer": {"heads": 2 * W // 64, "vdim": 64, "state": 128, "groups": 8,
+                     "norm_groups": 8, "conv": 4}}
+    layers = [par, lin, ssd, par] * depth_groups
+    return ModelConfig(arch="silonex", vocab_size=32000, hidden_size=W,
+                       num_hidden_layers=len(layers), rms_norm_eps=1e-6, streams=2,
+                       intermediate_size=0, num_attention_heads=0, num_key_value_heads=0,
+                       max_position_embeddings=1 << 20, eos_token_id=-1, tie_word_embeddings=True,
+                       name=f"silonex-w{W}", layer_specs=layers)
+
+
 def gedatar_attention_moe_config(width: int, depth: int = 4):
     """The closest older design at Fanopel's shapes: Gedatar attention layers (keys as values,
     chunk mask of 1024) with 16 gated experts of the same FFN width, top 4, no shared expert."""
@@ -224,7 +257,7 @@ def run_hybrid_bench(args) -> list:
     rows = []
     family = getattr(args, "hybrid_family", "gedatar")
     make = {"gedatar": gedatar_config, "dalavik": dalavik_config, "fanopel": fanopel_config,
-            "foderax": foderax_config}[family]
+            "foderax": foderax_config, "silonex": silonex_config}[family]
     for width in [int(w) for w in str(args.hybrid_widths).split(",")]:
         gcfg = make(width)
         beside = [llama_config(width, gcfg.num_hidden_layers)]
@@ -232,6 +265,8 @@ def run_hybrid_bench(args) -> list:
             beside.insert(0, gedatar_attention_moe_config(width, gcfg.num_hidden_layers))
         if family == "foderax":
             beside = [dalavik_config(width), fanopel_config(width, gcfg.num_hidden_layers)] + beside
+        if family == "silonex":
+            beside = [gedatar_config(width), fanopel_config(width, gcfg.num_hidden_layers)] + beside
         if getattr(args, "hybrid_only", False):
             beside = []
         for cfg in [gcfg] + beside:
@@ -255,8 +290,9 @@ def run_hybrid_bench(args) -> list:
             gd = by[(w, b, "gedatar")]
             row["prefill_vs_gedatar"] = round(r["prefill_tok_s"] / gd["prefill_tok_s"], 3)
             row["decode_vs_gedatar"] = round(r["decode_tok_s"] / gd["decode_tok_s"], 3)
-        if family == "foderax":
-            for other in ("dalavik", "fanopel"):
+        others = {"foderax": ("dalavik", "fanopel"), "silonex": ("gedatar", "fanopel")}
+        if family in others:
+            for other in others[family]:
                 o = by[(w, b, other)]
                 row[f"prefill_vs_{other}"] = round(r["prefill_tok_s"] / o["prefill_tok_s"], 3)
                 row[f"decode_vs_{other}"] = round(r["decode_tok_s"] / o["decode_tok_s"], 3)

@@ -41,7 +41,7 @@ def short_conv(x, taps, bias=None):
     start."""
     T, K = x.shape[0], taps.shape[1]
     y = torch.zeros_like(x)
-    for j in range(K):
+    for j in range(min(K, T)):
         y[j:] += taps[:, K - 1 - j] * x[:T - j]
     return y if bias is None else y + bias
 
@@ -69,7 +69,7 @@ def rotate_half_layout(x, rot):
     """x [T, n, D]: entry i pairs with entry i + dims / 2 (i < dims / 2); the rest passes."""
     T, half = x.shape[0], rot["dims"] // 2
     a = torch.arange(T, dtype=F64).view(T, 1, 1) * frequencies(rot).view(1, 1, -1)
-    c, s = torch.cos(a), torch.sin(a)
+    c, s = torch.cos(a).to(x.dtype), torch.sin(a).to(x.dtype)
     u, v = x[..., :half], x[..., half:2 * half]
     return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * half:]], -1)
 
@@ -103,7 +103,7 @@ def window_attention(h, w, p, m, eps):
 def delta_recurrence(q, k, v, beta, decay, S=None):
     """q, k [T, H, D] (one per head), v [T, H, Dv], beta, decay [T, H] -> (read-outs, state)."""
     T, H, D = q.shape
-    S = torch.zeros(H, D, v.shape[-1], dtype=F64) if S is None else S.clone()
+    S = torch.zeros(H, D, v.shape[-1], dtype=q.dtype) if S is None else S.clone()
     out = []
     for t in range(T):
         S = decay[t].view(H, 1, 1) * S
@@ -138,7 +138,7 @@ def parallel_mixer(h, w, p, m, eps):
 def decayed_recurrence(q, k, v, decay, S=None):
     """q, k [T, H, D], v [T, H, Dv], decay [T, H]: S <- decay S + k v^T, o = S^T q."""
     T, H, D = q.shape
-    S = torch.zeros(H, D, v.shape[-1], dtype=F64) if S is None else S.clone()
+    S = torch.zeros(H, D, v.shape[-1], dtype=q.dtype) if S is None else S.clone()
     out = []
     for t in range(T):
         S = decay[t].view(H, 1, 1) * S + k[t].unsqueeze(-1) * v[t].unsqueeze(1)
@@ -149,7 +149,7 @@ def decayed_recurrence(q, k, v, decay, S=None):
 def lightning(h, w, p, m, eps):
     T, H = h.shape[0], m["heads"]
     q, k, v = (silu(h @ w[p + n].T).view(T, H, -1) for n in "qkv")
-    decay = torch.tensor(m["decay"], dtype=F64).view(1, H).expand(T, H)
+    decay = torch.tensor(m["decay"], dtype=h.dtype).view(1, H).expand(T, H)
     o, _ = decayed_recurrence(q, k, v, decay)
     o = rms_unit(o.reshape(T, -1), eps) * w[p + "norm"] * torch.sigmoid(h @ w[p + "g"].T)
     return o @ w[p + "o"].T
@@ -215,10 +215,11 @@ def layer_order(cfg):
     return list(range(a)) + list(range(a, b)) * lp["times"] + list(range(b, n))
 
 
-def forward(cfg, weights, tokens, layers_out=None):
-    """Logits [T, vocab] (float64) of one sequence from position 0; ``layers_out`` (a list) takes
-    the sum of the streams after every layer run."""
-    w = {k: v.to(F64) for k, v in weights.items()}
+def forward(cfg, weights, tokens, layers_out=None, dtype=F64):
+    """Logits [T, vocab] of one sequence from position 0, computed in ``dtype`` (float32: what
+    rounding alone does to them); ``layers_out`` (a list) takes the sum of the streams after every
+    layer run."""
+    w = {k: v.to(dtype) for k, v in weights.items()}
     eps = cfg["norm"]["eps"]
     x = w["embed"][torch.as_tensor(tokens).long()]
     xs = x.unsqueeze(0).repeat(cfg.get("streams", 1), 1, 1)

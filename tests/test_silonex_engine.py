@@ -1,0 +1,609 @@
+"""Silonex through the serving engine (model registry, loader, block manager, state slots,
+scheduler, hybrid runner, trace replay) against the float64 whole-sequence oracle of
+tests/_ref_silonex.py.
+
+Every test runs on the CPU (the ops' torch path) and, marked ``gpu``, on the HIP kernels.  The
+configurations are small and unlike each other: head sizes that are and are not multiples of the
+vector and matrix-core widths, grouped, multi-query and full heads, rotary on a part of the head
+and on all of it, one to four residual copies, loops at the start, in the middle and over the
+whole stack, one tap and many, one head, layers without a feed-forward, stacks that begin with
+each kind of layer."""
+import copy
+import os
+
+import pytest
+import torch
+
+import _ref_silonex as ref
+from test_foderax_engine import _NoTokenizer, check, check_rounding, engine, replay_alone, tokens
+
+from lumen.models import build_model
+from lumen.models.config import ModelConfig, get_config, silonex_to_dict
+from lumen.models.silonex import SilonexForCausalLM
+from lumen.serve.hybrid_runner import key_bytes_per_token, state_bytes_per_slot
+from lumen.serve.sequence import SamplingParams
+from lumen.serve.trace import TraceReplay
+
+DEVICES = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
+assert _NoTokenizer is not None
+
+
+def _cfg(name, vocab, width, streams, loop, logit_scale, eps, layers):
+    return ModelConfig(arch="silonex", vocab_size=vocab, hidden_size=width, streams=streams,
+                       loop=loop, logit_scale=logit_scale, num_hidden_layers=len(layers),
+                       rms_norm_eps=eps, intermediate_size=0, num_attention_heads=0,
+                       num_key_value_heads=0, max_position_embeddings=1 << 20, eos_token_id=-1,
+                       tie_word_embeddings=True, name=name, layer_specs=layers)
+
+
+def _ff(n):
+    return {"kind": "dense", "ff": n} if n else None
+
+
+def _par(left, right, ff, window, cap=12.0, scaling="default", base=3000.0, scale=0.3):
+    H, G, D, Dv, rot = left
+    r = {"base": base, "dims": rot}
+    if scaling == "default":
+        r["scaling"] = {"factor": 4.0, "low": 1.0, "high": 4.0, "original": 128}
+    elif scaling:
+        r["scaling"] = scaling
+    m = {"heads": H, "kv_heads": G, "dim": D, "vdim": Dv, "scale": scale, "rot": r,
+         "mask": {"size": window}}
+    if cap:
+        m["softcap"] = cap
+    h, g, d, dv, conv = right
+    return {"type": "parallel", "mlp": _ff(ff), "mixer": {
+        "left": m, "right": {"heads": h, "kv_heads": g, "dim": d, "vdim": dv, "conv": conv}}}
+
+
+def _lin(H, D, Dv, decay, ff):
+    return {"type": "lightning", "mlp": _ff(ff),
+            "mixer": {"heads": H, "dim": D, "vdim": Dv, "decay": decay}}
+
+
+def _ssd(H, P, N, G, norm_groups, conv, ff):
+    return {"type": "mamba2", "mlp": _ff(ff), "mixer": {
+        "heads": H, "vdim": P, "state": N, "groups": G, "norm_groups": norm_groups, "conv": conv}}
+
+
+CONFIGS = {
+    "tiny": lambda: copy.deepcopy(get_config("tiny-silonex")),
+    # nothing a multiple of 8: scalar paths everywhere; full-head attention beside multi-query delta
+    # heads; three loops over the first two layers; one tap; a stack that starts with state-space
+    # duality; layers without a feed-forward; no soft cap, no frequency stretching
+    "odd": lambda: _cfg("odd", 131, 60, 3, {"start": 0, "stop": 2, "times": 3}, 0.7, 3e-6, [
+        _ssd(3, 10, 6, 1, 5, 3, 28),
+        _par((3, 3, 10, 14, 6), (3, 1, 9, 11, 1), None, 21, cap=None, scaling=None),
+        _lin(3, 11, 7, [0.3, 1.0, 0.97], 33),
+        _ssd(2, 5, 37, 2, 1, 5, None)]),
+    # one of everything: one copy, one head, one group, no loop, a window of one token, a factor of 1
+    "one": lambda: _cfg("one", 64, 48, 1, None, 1.0, 1e-4, [
+        _lin(1, 16, 16, [0.9], 40),
+        _par((1, 1, 16, 16, 16), (1, 1, 16, 16, 2), 24, 1),
+        _ssd(1, 16, 16, 1, 1, 2, 24)]),
+    # head sizes 64 and 128 (the matrix-core attention's shapes), wide states, four copies, the whole
+    # stack looped, a window across tiles
+    "wide": lambda: _cfg("wide", 200, 128, 4, {"start": 0, "stop": 3, "times": 2}, 2.5, 1e-5, [
+        _par((4, 1, 64, 64, 64), (2, 1, 128, 128, 4), 160, 70, base=500000.0, scale=0.12),
+        _ssd(4, 64, 128, 1, 4, 4, 96),
+        _lin(2, 128, 64, [0.8, 0.995], None)]),
+}
+
+
+def make(name, device, dtype=torch.float32, seed=0):
+    m = SilonexForCausalLM(CONFIGS[name](), dtype=dtype, device=device)
+    m.init_weights(seed=seed)
+    return m
+
+
+class Oracle:
+    def __init__(self, model):
+        self.cfg = silonex_to_dict(model.config)
+        self.w = {n: model.tensor(n).detach().cpu() for n in model.tensor_names()}
+
+    def forward(self, toks, cfg=None, w=None, dtype=ref.F64):
+        return ref.forward(cfg or self.cfg, w or self.w, toks, dtype=dtype)
+
+
+oracle = Oracle
+
+
+def yardstick(orc, toks, want):
+    """[T] what rounding to fp32 alone does to each position's logits: the oracle's own arithmetic in
+    fp32 against float64.  A norm over a read-out that happens to be nearly zero magnifies rounding
+    at that position a thousandfold, in any implementation."""
+    return (orc.forward(toks, dtype=torch.float32).to(ref.F64) - want).abs().max(-1).values
+
+
+def check_conditioned(got, want, stick, rtol=2e-4):
+    """``check``, with positions that rounding alone moves allowed a multiple of that."""
+    per = (got.to(ref.F64) - want).abs().max(-1).values
+    limit = torch.clamp(8.0 * stick, min=rtol * max(float(want.std()), 1.0))
+    t = int((per / limit).argmax())
+    assert float(per[t]) <= float(limit[t]), f"position {t}: {float(per[t]):.3e} > {float(limit[t]):.3e}"
+    assert int((stick > rtol).sum()) <= 4, "the weights make most positions ill-conditioned"
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_whole_prompt_matches_oracle(device, name):
+    m = make(name, device)
+    toks = tokens(m, 150, 1)
+    want = oracle(m).forward(toks)
+    check(replay_alone(m, device, toks, [1000]), want)
+    # the model's own forward (fresh caches, every row) is the same step function
+    check(m(torch.tensor(toks, device=device))[0].cpu(), want)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_stream_after_every_pass(device, name):
+    """The runner's per-layer hook against the oracle's sum of the copies after every pass of a
+    layer: a fault shows at its layer."""
+    m = make(name, device, seed=13)
+    toks = tokens(m, 29, 14)
+    layers = []
+    o = oracle(m)
+    ref.forward(o.cfg, o.w, toks, layers)
+    eng = engine(m, device)
+    seen = {}
+    eng.runner.observe = lambda i, x: seen.__setitem__(i, x.detach().float().cpu().clone())
+    TraceReplay(eng).step([{"id": "a", "tokens": toks, "want": []}], ["a"])
+    assert sorted(seen) == list(range(len(layers)))
+    for i, want in enumerate(layers):
+        err = float((seen[i].to(ref.F64) - want).abs().max())
+        assert err <= 1e-4 * max(1.0, float(want.abs().max())), f"pass {i}: {err:.3e}"
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_prefill_then_long_decode(device, name):
+    """A short prompt, then token by token across block, tile and chunk borders: states, tails and
+    caches carried from step to step."""
+    m = make(name, device, seed=1)
+    toks = tokens(m, 170, 2)
+    want = oracle(m).forward(toks)
+    check(replay_alone(m, device, toks, [5] + [1] * 300), want)
+    # from the very first token on, one at a time (the first token is a one-row prefill)
+    check(replay_alone(m, device, toks[:40], [1]), want[:40])
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("pieces", [[2], [3, 1, 2, 17, 2, 1, 1, 30], [16], [15, 1, 17], [64, 2, 63],
+                                    [33, 2], [129, 2]])
+def test_portions_of_several_sizes(device, pieces):
+    m = make("tiny", device, seed=2)
+    toks = tokens(m, 137, 3)
+    check(replay_alone(m, device, toks, pieces, bs=8), oracle(m).forward(toks))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_long_portions_carry_state(device):
+    """Portions longer than the scans' chunks, cut off the chunk grid."""
+    m = make("odd", device, seed=12)
+    toks = tokens(m, 330, 4)
+    orc = oracle(m)
+    want = orc.forward(toks)
+    stick = yardstick(orc, toks, want)
+    check_conditioned(replay_alone(m, device, toks, [1000]), want, stick)
+    check_conditioned(replay_alone(m, device, toks, [197, 1, 130, 2]), want, stick)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_first_tokens(device, name):
+    m = make(name, device, seed=3)
+    orc = oracle(m)
+    for n in (1, 2, 3, 6):
+        toks = tokens(m, n, 10 + n)
+        check(replay_alone(m, device, toks, [1000]), orc.forward(toks))
+        check(replay_alone(m, device, toks, [1]), orc.forward(toks))
+
+
+def _sharpen(m, factor=4.0):
+    """Scale the attention halves' query weights up: a few keys, wherever they lie, carry a row's
+    weight, so that a window that is one token off or a wrong key shows."""
+    with torch.no_grad():
+        for i, L in enumerate(m.config.layer_specs):
+            if L["type"] == "parallel":
+                m.tensor(f"l{i}.mix.left.q.norm").mul_(factor)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name", ["tiny", "wide"])
+def test_every_constant_counts(device, name):
+    """Sharp scores.  The oracle itself says that a window one token off, a missing soft cap, the
+    plain frequencies, another loop count, another norm grouping, a dropped skip, a mixing matrix
+    read as [to, from], a decay or a step bias that is off, a dropped convolution bias, a factor of
+    1 on the logits ... would move the logits far beyond the tolerance -- and the engine matches
+    the true model whole, in ragged portions and decoded token by token."""
+    m = make(name, device, seed=21)
+    _sharpen(m)
+    toks = tokens(m, 160, 22)
+    orc = oracle(m)
+    want = orc.forward(toks)
+    scale = max(float(want.std()), 1.0)
+    kinds = [L["type"] for L in orc.cfg["layers"]]
+    ip, il, im = kinds.index("parallel"), kinds.index("lightning"), kinds.index("mamba2")
+
+    def cfg_with(fn):
+        c = copy.deepcopy(orc.cfg)
+        fn(c)
+        return c, None
+
+    def w_with(name_, fn):
+        w = dict(orc.w)
+        w[name_] = fn(w[name_].float()).to(w[name_].dtype)
+        return None, w
+
+    def left(c):
+        return c["layers"][ip]["mixer"]["left"]
+
+    def set_(d, k, v):
+        d[k] = v
+
+    right, ssd = f"l{ip}.mix.right.", f"l{im}.mix."
+    changes = {
+        "window + 1": cfg_with(lambda c: set_(left(c)["mask"], "size", left(c)["mask"]["size"] + 1)),
+        "window - 1": cfg_with(lambda c: set_(left(c)["mask"], "size", left(c)["mask"]["size"] - 1)),
+        "soft cap": cfg_with(lambda c: set_(left(c), "softcap", None)),
+        "stretch": cfg_with(lambda c: set_(left(c)["rot"], "scaling", None)),
+        "scale": cfg_with(lambda c: set_(left(c), "scale", left(c)["scale"] * 0.9)),
+        "loop": cfg_with(lambda c: set_(c["loop"], "times", c["loop"]["times"] + 1)),
+        "norm groups": cfg_with(lambda c: set_(
+            c["layers"][im]["mixer"], "norm_groups", 1)),
+        "lightning decay": cfg_with(lambda c: set_(
+            c["layers"][il]["mixer"], "decay", [d * 0.95 for d in c["layers"][il]["mixer"]["decay"]])),
+        "logit scale": cfg_with(lambda c: set_(c, "logit_scale", 1.0)),
+        "skip": w_with(ssd + "D", lambda t: t * 0.0),
+        "ssd decay": w_with(ssd + "A_log", lambda t: t + 0.3),
+        "ssd step bias": w_with(ssd + "dt_bias", lambda t: t * 0.0),
+        "conv bias": w_with(ssd + "conv.b", lambda t: t * 0.0),
+        "conv order": w_with(ssd + "conv", lambda t: t.flip(1)),
+        "delta decay": w_with(right + "A_log", lambda t: t + 0.3),
+        "delta step bias": w_with(right + "dt_bias", lambda t: t * 0.0),
+        "delta conv order": w_with(right + "k.conv", lambda t: t.flip(1)),
+        "beta": w_with(right + "b", lambda t: t * 0.0),
+        "output norm": w_with(right.replace("right", "left") + "out", lambda t: t * 0.0 + 1.0),
+        "mix": w_with(f"l{ip}.hc1.mix", lambda t: t.t().contiguous()),
+        "in": w_with(f"l{ip}.hc1.in", lambda t: t * 0.0 + 1.0 / t.numel()),
+        "out": w_with(f"l{ip}.hc1.out", lambda t: t.flip(0)),
+        "shift": w_with(f"l{ip}.norm1.b", lambda t: t * 0.0),
+    }
+    for what, (c, w) in changes.items():
+        moved = float((orc.forward(toks, c, w) - want).abs().max())
+        assert moved > 20 * 5e-4 * scale, f"{what}: moves the logits by {moved:.2e} only"
+    check(replay_alone(m, device, toks, [1000]), want, rtol=5e-4)
+    check(replay_alone(m, device, toks, [37, 2, 50, 1, 64, 3], bs=8), want, rtol=5e-4)
+    check(replay_alone(m, device, toks, [90] + [1] * 200), want, rtol=5e-4)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_far_token_is_seen(device):
+    """Changing the FIRST token of a long prompt changes the last logits only through the states
+    (the window has passed it long ago); the engine agrees with the oracle on both prompts."""
+    m = make("tiny", device, seed=23)
+    with torch.no_grad():                                     # slow decays: the first write lasts
+        for i, L in enumerate(m.config.layer_specs):
+            for part in {"parallel": ["right."], "mamba2": [""]}.get(L["type"], []):
+                m.tensor(f"l{i}.mix.{part}A_log").fill_(-6.0)
+    m.config.layer_specs[0]["mixer"]["decay"] = [0.999, 0.9995, 1.0]
+    orc = oracle(m)
+    a = tokens(m, 260, 24)
+    b = list(a)
+    b[0] = (a[0] + 1) % m.config.vocab_size
+    wa, wb = orc.forward(a)[-1], orc.forward(b)[-1]
+    assert float((wa - wb).abs().max()) > 20 * 5e-4 * float(wa.std())
+    for toks, want in ((a, wa), (b, wb)):
+        check(replay_alone(m, device, toks, [230, 7, 1], bs=8)[-1:], want[None], rtol=5e-4)
+        check(replay_alone(m, device, toks, [200] + [1] * 60, bs=8)[-1:], want[None], rtol=5e-4)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name", ["tiny", "odd"])
+def test_mixed_batches_reuse_blocks_and_slots(device, name):
+    """Seven unequal requests through three sequence slots and a pool of 20 blocks of 8: portions
+    of some beside single tokens of others; finished requests hand their blocks and their state
+    slot (with states and convolution tails still in it) to new ones.  Every request must come out
+    as if it had run alone."""
+    m = make(name, device, seed=4)
+    orc = oracle(m)
+    lens = [41, 9, 66, 2, 30, 17, 50]
+    reqs = {f"r{i}": tokens(m, n, 20 + i) for i, n in enumerate(lens)}
+    eng = engine(m, device, blocks=20, bs=8, seqs=3)
+    rp = TraceReplay(eng)
+    g = torch.Generator().manual_seed(5)
+    waiting = list(reqs)
+    live, at, got = [], {}, {r: [] for r in reqs}
+    sizes = [2, 1, 1, 13, 1, 5, 1, 1, 24, 3]
+    k = 0
+    seen_blocks, seen_slots = [], []
+    while waiting or live:
+        while waiting and len(live) < 3:
+            need = sum((len(reqs[r]) + 7) // 8 for r in live + [waiting[0]])
+            if need > 20:
+                break
+            r = waiting.pop(0)
+            live.append(r)
+            at[r] = 0
+        entries, end = [], []
+        for r in list(live):
+            if len(live) > 1 and torch.rand((), generator=g) < 0.3:
+                continue                                   # left out of this step
+            c = min(sizes[k % len(sizes)], len(reqs[r]) - at[r])
+            k += 1
+            entries.append({"id": r, "tokens": reqs[r][at[r]:at[r] + c], "want": list(range(c))})
+            at[r] += c
+            if at[r] == len(reqs[r]):
+                end.append(r)
+                live.remove(r)
+        if not entries:
+            continue
+        seen_slots += list(eng.states.owner.values())
+        out = rp.step(entries, end)
+        seen_blocks += [b for t in eng.blocks.tables.values() for b in t]
+        o = 0
+        for e in entries:
+            got[e["id"]].append(out[o:o + len(e["tokens"])])
+            o += len(e["tokens"])
+    assert eng.blocks.num_free == 20 and len(set(seen_blocks)) <= 20
+    assert eng.states.num_free == 3 and set(seen_slots) <= {0, 1, 2}
+    for r, toks in reqs.items():
+        check(torch.cat(got[r], 0), orc.forward(toks))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name", ["tiny", "odd"])
+def test_blocks_and_slot_reused_after_finish(device, name):
+    """The second request gets the first one's blocks and state slot, full of its keys, values,
+    states and tails."""
+    m = make(name, device, seed=6)
+    orc = oracle(m)
+    eng = engine(m, device, blocks=8, bs=16, seqs=1)
+    rp = TraceReplay(eng)
+    a, b = tokens(m, 100, 30), tokens(m, 60, 31)
+    rp.step([{"id": "a", "tokens": a, "want": []}], ["a"])
+    got = torch.cat([rp.step([{"id": "b", "tokens": b[:1], "want": [0]}], []),
+                     rp.step([{"id": "b", "tokens": b[1:33], "want": list(range(32))}], []),
+                     rp.step([{"id": "b", "tokens": b[33:], "want": list(range(27))}], ["b"])], 0)
+    check(got, orc.forward(b))
+
+
+def test_every_pass_has_caches_of_its_own():
+    """A looped layer's passes must not share memory, and the byte counts follow the passes."""
+    m = make("tiny", "cpu")
+    eng = engine(m, "cpu", blocks=4, bs=8, seqs=2)
+    st = eng.runner.state
+    runs = eng.weights.runs
+    assert runs == [0, 1, 2, 1, 2, 3]
+    ptrs = [t.data_ptr() for group in (st.k, st.v, st.S, st.tail) for t in group if t is not None]
+    assert len(ptrs) == len(set(ptrs))
+    per_tok = sum(t[0, 0].numel() for g in (st.k, st.v) for t in g if t is not None) * 4
+    assert key_bytes_per_token(m.config, 4) == per_tok
+    per_slot = sum(t[0].numel() for g in (st.S, st.tail) for t in g if t is not None) * 4
+    assert state_bytes_per_slot(m.config, 4) == per_slot
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("name", ["tiny", "one"])
+def test_greedy_generation_through_scheduler(device, name):
+    """LLMEngine.generate: chunked prefill under a small token budget, more prompts than
+    sequence slots, async scheduling, greedy sampling -- every generated token is the oracle's
+    arg-max (up to a tie within the tolerance) given the tokens before it."""
+    m = make(name, device, seed=7)
+    orc = oracle(m)
+    eng = engine(m, device, blocks=48, bs=8, seqs=3, budget=24)
+    prompts = [tokens(m, n, 40 + n) for n in (5, 37, 1, 20, 52)]
+    seqs = eng.generate(prompts, SamplingParams(max_tokens=10, temperature=0.0, ignore_eos=True))
+    assert eng.blocks.num_free == 48 and eng.states.num_free == 3
+    for p, s in zip(prompts, seqs):
+        assert len(s.output_ids) == 10
+        want = orc.forward(p + s.output_ids[:-1])
+        for j, tok in enumerate(s.output_ids):
+            row = want[len(p) - 1 + j]
+            assert float(row.max() - row[tok]) <= 1e-3 * max(float(row.std()), 1.0)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_preemption_recomputes_caches_and_state(device):
+    """A pool too small for all running sequences: the scheduler preempts and later recomputes a
+    sequence from its first token in whatever blocks and slot it then gets; outputs stay the
+    oracle's."""
+    m = make("odd", device, seed=8)
+    orc = oracle(m)
+    eng = engine(m, device, blocks=12, bs=4, seqs=3, budget=64, async_scheduling=False)
+    prompts = [tokens(m, n, 60 + n) for n in (9, 11, 10)]
+    seqs = eng.generate(prompts, SamplingParams(max_tokens=14, temperature=0.0, ignore_eos=True))
+    assert eng.scheduler.num_preemptions > 0
+    for p, s in zip(prompts, seqs):
+        want = orc.forward(p + s.output_ids[:-1])
+        for j, tok in enumerate(s.output_ids):
+            row = want[len(p) - 1 + j]
+            assert float(row.max() - row[tok]) <= 1e-3 * max(float(row.std()), 1.0)
+
+
+def _random_config(seed):
+    """A random stack: 1 - 5 layers in random order with a random loop, sizes that are and are not
+    multiples of the vector and matrix-core widths."""
+    import random
+
+    rng = random.Random(seed)
+    W = rng.choice([64, 96, 160, 192])
+    layers = []
+    for _ in range(rng.randint(1, 5)):
+        ff = rng.choice([None, 40, 92, 128])
+        kind = rng.choice(["parallel", "parallel", "lightning", "mamba2"])
+        H = rng.choice([1, 2, 3, 4, 6, 8])
+        G = rng.choice([g for g in (1, 2, 3, 4, H) if H % g == 0])
+        D, Dv = rng.choice([8, 12, 20, 32, 64]), rng.choice([8, 12, 24, 32, 64, 72])
+        if kind == "parallel":
+            h = rng.choice([1, 2, 4, 6])
+            g = rng.choice([x for x in (1, 2, 3) if h % x == 0])
+            layers.append(_par((H, G, D, Dv, rng.choice([2, D // 4 * 2, D])),
+                               (h, g, rng.choice([8, 17, 32, 64]), rng.choice([8, 20, 32, 48]),
+                                rng.choice([1, 2, 3, 4])), ff, rng.choice([1, 5, 32, 50, 129]),
+                               cap=rng.choice([5.0, 20.0]), base=rng.choice([100.0, 10000.0]),
+                               scale=rng.uniform(0.1, 0.6)))
+        elif kind == "lightning":
+            layers.append(_lin(H, D, Dv, [rng.choice([0.4, 0.9, 0.99, 1.0]) for _ in range(H)], ff))
+        else:
+            n = rng.choice([x for x in (1, 2, 3, 4) if (H * Dv) % x == 0])
+            layers.append(_ssd(H, Dv, rng.choice([8, 16, 36, 64]), G, n, rng.choice([2, 3, 4, 6]), ff))
+    a = rng.randint(0, len(layers) - 1)
+    loop = {"start": a, "stop": rng.randint(a, len(layers)), "times": rng.randint(1, 3)}
+    return _cfg(f"random{seed}", rng.randint(50, 400), W, rng.choice([1, 2, 3, 4]),
+                rng.choice([None, loop]), rng.choice([0.5, 1.0, 3.0]), rng.choice([1e-6, 1e-5]), layers)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("seed", range(10))
+def test_random_configurations(device, seed):
+    """Whole, in ragged portions, and decoded across a tile border: the oracle's logits (fp32)
+    and, on the GPU in 16 bits, the same logits however the prompt was cut."""
+    cfg = _random_config(seed)
+    m = SilonexForCausalLM(cfg, dtype=torch.float32, device=device)
+    m.init_weights(seed=seed)
+    toks = tokens(m, 150, seed)
+    orc = oracle(m)
+    want = orc.forward(toks)
+    stick = yardstick(orc, toks, want)
+    for pieces in ([1000], [37, 2, 1, 50, 1, 1, 1, 3], [120] + [1] * 30):
+        check_conditioned(replay_alone(m, device, toks, pieces), want, stick)
+    if device == "cuda":
+        m16 = SilonexForCausalLM(cfg, dtype=torch.bfloat16, device=device)
+        m16.init_weights(seed=seed)
+        whole = replay_alone(m16, device, toks, [1000])
+        check_rounding(replay_alone(m16, device, toks, [37, 2, 1, 50, 1, 1, 1, 3]), whole)
+        check_rounding(replay_alone(m16, device, toks, [120] + [1] * 30), whole)
+
+
+def test_configuration_is_validated():
+    def bad(fn, name="odd"):
+        c = CONFIGS[name]()
+        fn(c)
+        with pytest.raises(ValueError):
+            SilonexForCausalLM(c, dtype=torch.float32, device="cpu")
+
+    mixer = lambda c, i: c.layer_specs[i]["mixer"]  # noqa: E731
+    bad(lambda c: mixer(c, 1)["left"].update(kv_heads=2))     # 3 heads on 2 key heads
+    bad(lambda c: mixer(c, 1)["right"].update(kv_heads=2))
+    bad(lambda c: mixer(c, 1)["left"]["rot"].update(dims=7))
+    bad(lambda c: mixer(c, 1)["right"].update(dim=300))       # a state row the scan has no kernel for
+    bad(lambda c: mixer(c, 1)["right"].update(conv=0))
+    bad(lambda c: mixer(c, 0).update(groups=2))               # 3 heads in 2 groups
+    bad(lambda c: mixer(c, 0).update(norm_groups=4))          # 30 channels in 4 parts
+    bad(lambda c: mixer(c, 2).update(decay=[0.5]))            # 3 heads
+    bad(lambda c: c.loop.update(stop=9))
+    bad(lambda c: c.loop.update(times=0))
+    bad(lambda c: setattr(c, "streams", 0))
+    bad(lambda c: setattr(c, "streams", 9))
+    bad(lambda c: c.layer_specs[0].update(type="window"))
+    bad(lambda c: c.layer_specs[0].update(mlp={"kind": "moe"}))
+
+
+def test_checkpoint_roundtrip(tmp_path):
+    """save -> config.json + model.safetensors under the design's tensor names -> load by
+    directory (the class is picked by config.json); a missing tensor or a wrong shape is an
+    error."""
+    from safetensors.torch import load_file, save_file
+
+    from lumen.models.loading import save_hf_weights
+
+    for name in ("one", "odd"):
+        m = make(name, "cpu", dtype=torch.bfloat16)
+        d = str(tmp_path / name)
+        save_hf_weights(m, d)
+        m2 = build_model(d, dtype=torch.bfloat16, device="cpu")
+        assert m2.config.arch == "silonex" and type(m2) is SilonexForCausalLM
+        for f in ("streams", "loop", "logit_scale", "layer_specs", "rms_norm_eps"):
+            assert getattr(m2.config, f) == getattr(m.config, f), f
+        for n in m.tensor_names():
+            assert torch.equal(m.tensor(n), m2.tensor(n)), n
+    f = os.path.join(d, "model.safetensors")
+    sd = load_file(f)
+    assert "l1.norm2" not in sd and "l1.hc2.mix" not in sd      # a layer without a feed-forward
+    short = dict(sd)
+    short.pop("l1.mix.right.k.conv")
+    save_file(short, f)
+    with pytest.raises(KeyError):
+        build_model(d, dtype=torch.bfloat16, device="cpu")
+    sd["l0.hc1.mix"] = torch.zeros(2, 3, dtype=torch.bfloat16)
+    save_file(sd, f)
+    with pytest.raises(ValueError):
+        build_model(d, dtype=torch.bfloat16, device="cpu")
+
+
+def test_trace_run_command_line(tmp_path):
+    """bin/trace_run as a user runs it: a checkpoint directory, JSON steps on stdin, one logits
+    file per step that wants any, `done <step>` after every step, exit code 0 at end of input."""
+    import json
+    import subprocess
+    import sys
+
+    import numpy as np
+
+    from lumen.models.loading import save_hf_weights
+
+    m = make("odd", "cpu", dtype=torch.bfloat16)
+    d = str(tmp_path / "ckpt")
+    out = str(tmp_path / "out")
+    save_hf_weights(m, d)
+    a, b = tokens(m, 21, 70), tokens(m, 12, 71)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:9], "want": [0, 8]}], "end": []},
+             {"step": 1, "entries": [{"id": "a", "tokens": a[9:10], "want": []},
+                                     {"id": "b", "tokens": b[:11], "want": [10]}], "end": []},
+             {"step": 2, "entries": [{"id": "b", "tokens": b[11:], "want": [0]},
+                                     {"id": "a", "tokens": a[10:], "want": [10]}],
+              "end": ["a", "b"]}]
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    r = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", d,
+                        "--dtype", "float32", "--out", out, "--max-tokens", "128", "--device", "cpu"],
+                       input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True,
+                       text=True, timeout=300)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [ln for ln in r.stdout.splitlines() if ln.startswith("done")] == ["done 0", "done 1", "done 2"]
+    orc = oracle(m)
+    ra, rb = orc.forward(a), orc.forward(b)
+    V = m.config.vocab_size
+    got = {i: torch.from_numpy(np.fromfile(os.path.join(out, f"{i}.f32"), dtype="<f4")).view(-1, V)
+           for i in range(3)}
+    check(got[0], ra[[0, 8]])
+    check(got[1], rb[[10]])
+    check(got[2], torch.stack([rb[11], ra[20]]))
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_bf16_close_to_oracle_and_cut_invariant(name):
+    """bf16 serving: within rounding of the float64 oracle, and the same logits (to rounding)
+    however the prompt is cut and whether rows decode through the hipGraph path or eagerly."""
+    m = make(name, "cuda", dtype=torch.bfloat16, seed=9)
+    toks = tokens(m, 170, 50)
+    want = oracle(m).forward(toks)
+    whole = replay_alone(m, "cuda", toks, [1000])
+    cut = replay_alone(m, "cuda", toks, [7, 1, 2, 1, 1, 16])
+    eager = replay_alone(m, "cuda", toks, [30] + [1] * 150, graphs=False)
+    for got in (whole, cut, eager):
+        check_rounding(got, want)
+    check_rounding(cut, whole)
+
+
+@pytest.mark.gpu
+def test_graph_replayed_decode_matches_eager():
+    """Decode steps replay a captured hipGraph per batch bucket; several replays, with eager
+    prefill steps of other requests between them, give what eager decoding gives."""
+    m = make("tiny", "cuda", seed=10)
+    a, b = tokens(m, 50, 51), tokens(m, 33, 52)
+    wa, wb = oracle(m).forward(a), oracle(m).forward(b)
+    rp = TraceReplay(engine(m, "cuda", graphs=True))
+    got_a = [rp.step([{"id": "a", "tokens": a[:20], "want": list(range(20))}], [])]
+    for i in range(20, 35):                                # graph bucket 1
+        got_a.append(rp.step([{"id": "a", "tokens": a[i:i + 1], "want": [0]}], []))
+    got_b = [rp.step([{"id": "b", "tokens": b[:10], "want": list(range(10))}], [])]
+    for i in range(15):                                    # graph bucket 2, both decoding
+        o = rp.step([{"id": "a", "tokens": a[35 + i:36 + i], "want": [0]},
+                     {"id": "b", "tokens": b[10 + i:11 + i], "want": [0]}], [])
+        got_a.append(o[0:1])
+        got_b.append(o[1:2])
+    check(torch.cat(got_a, 0), wa)
+    check(torch.cat(got_b, 0), wb[:25])
