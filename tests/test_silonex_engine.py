@@ -15,7 +15,7 @@ import pytest
 import torch
 
 import _ref_silonex as ref
-from test_foderax_engine import _NoTokenizer, check, check_rounding, engine, replay_alone, tokens
+from test_foderax_engine import check, engine, replay_alone, tokens
 
 from lumen.models import build_model
 from lumen.models.config import ModelConfig, get_config, silonex_to_dict
@@ -25,7 +25,6 @@ from lumen.serve.sequence import SamplingParams
 from lumen.serve.trace import TraceReplay
 
 DEVICES = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
-assert _NoTokenizer is not None
 
 
 def _cfg(name, vocab, width, streams, loop, logit_scale, eps, layers):
@@ -121,7 +120,23 @@ def check_conditioned(got, want, stick, rtol=2e-4):
     limit = torch.clamp(8.0 * stick, min=rtol * max(float(want.std()), 1.0))
     t = int((per / limit).argmax())
     assert float(per[t]) <= float(limit[t]), f"position {t}: {float(per[t]):.3e} > {float(limit[t]):.3e}"
-    assert int((stick > rtol).sum()) <= 4, "the weights make most positions ill-conditioned"
+    assert float((stick > rtol).double().mean()) <= 0.1, "the weights make most rows ill-conditioned"
+
+
+def close_to_rounding(m, toks, want, *gots):
+    """16-bit serving: every result's error (per position, root mean square over the logits) against
+    what 16-bit storage alone does, measured on the ops' torch path: typical and unusual positions
+    both within a factor of it, and the results as close to each other."""
+    twin = SilonexForCausalLM(m.config, dtype=m.dtype, device="cpu")
+    for n in m.tensor_names():
+        twin.tensor(n).data.copy_(m.tensor(n).cpu())
+    rms = lambda a, b: (a.to(ref.F64) - b.to(ref.F64)).pow(2).mean(-1).sqrt()  # noqa: E731
+    stick = rms(twin(torch.tensor(toks))[0], want)
+    for a, b in [(g, want) for g in gots] + [(g, gots[0]) for g in gots[1:]]:
+        per = rms(a, b)
+        for q in (0.5, 0.95):
+            e, s = float(per.quantile(q)), float(stick.quantile(q))
+            assert e <= (1.5 if q == 0.5 else 2.5) * s, f"quantile {q}: {e:.3e} against {s:.3e}"
 
 
 @pytest.mark.parametrize("device", DEVICES)
@@ -162,10 +177,12 @@ def test_prefill_then_long_decode(device, name):
     caches carried from step to step."""
     m = make(name, device, seed=1)
     toks = tokens(m, 170, 2)
-    want = oracle(m).forward(toks)
-    check(replay_alone(m, device, toks, [5] + [1] * 300), want)
+    orc = oracle(m)
+    want = orc.forward(toks)
+    stick = yardstick(orc, toks, want)
+    check_conditioned(replay_alone(m, device, toks, [5] + [1] * 300), want, stick)
     # from the very first token on, one at a time (the first token is a one-row prefill)
-    check(replay_alone(m, device, toks[:40], [1]), want[:40])
+    check_conditioned(replay_alone(m, device, toks[:40], [1]), want[:40], stick[:40])
 
 
 @pytest.mark.parametrize("device", DEVICES)
@@ -473,8 +490,9 @@ def test_random_configurations(device, seed):
         m16 = SilonexForCausalLM(cfg, dtype=torch.bfloat16, device=device)
         m16.init_weights(seed=seed)
         whole = replay_alone(m16, device, toks, [1000])
-        check_rounding(replay_alone(m16, device, toks, [37, 2, 1, 50, 1, 1, 1, 3]), whole)
-        check_rounding(replay_alone(m16, device, toks, [120] + [1] * 30), whole)
+        close_to_rounding(m16, toks, oracle(m16).forward(toks), whole,
+                          replay_alone(m16, device, toks, [37, 2, 1, 50, 1, 1, 1, 3]),
+                          replay_alone(m16, device, toks, [120] + [1] * 30))
 
 
 def test_configuration_is_validated():
@@ -583,9 +601,7 @@ def test_bf16_close_to_oracle_and_cut_invariant(name):
     whole = replay_alone(m, "cuda", toks, [1000])
     cut = replay_alone(m, "cuda", toks, [7, 1, 2, 1, 1, 16])
     eager = replay_alone(m, "cuda", toks, [30] + [1] * 150, graphs=False)
-    for got in (whole, cut, eager):
-        check_rounding(got, want)
-    check_rounding(cut, whole)
+    close_to_rounding(m, toks, want, whole, cut, eager)
 
 
 @pytest.mark.gpu
