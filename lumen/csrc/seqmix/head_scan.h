@@ -42,4 +42,14 @@ __device__ __forceinline__ void head_decay(const HeadScanArgs<T>& s, long long r
   ld = fmaxf(ld, -1e4f);
 }
 
+// silu of a stored q or k element, rounded to its type again: what a projection with an activation
+// stores, so that every kernel multiplies the same values
+template <typename T> __device__ __forceinline__ float silu_stored(float x) {
+  return to_f32(from_f32<T>(silu_f(x)));
+}
+
+// bf16 prompt portions (head_scan_chunk16.hip)
+hipError_t head_scan_chunk16(const HeadScanArgs<bf16>& args, bool delta, int n_seg,
+                             hipStream_t st);
+
 }  // namespace lumen

@@ -17,8 +17,8 @@
 // register r IS the right operand of one k = 2 product over the inner pair {a, a + 4}, when the
 // left operand is read as [row][a + 4 hi].  So state and U never pass through LDS; the left
 // operands (Q, K, the two chunk matrices) are staged there once for all waves and read 16 bytes at
-// a time.  The products are fp32 matrix instructions (fp32 in, fp32 accumulate): the same
-// arithmetic serves 16-bit and fp32 models.  Log-decay sums and their differences are fp64, so
+// a time.  The products are fp32 matrix instructions (fp32 in, fp32 accumulate); bf16 models take
+// head_scan_chunk16.hip instead.  Log-decay sums and their differences are fp64, so
 // G is accurate however far a chunk decays.
 // State in HBM: [slot][head][Dk][Dv] fp32; a segment that starts at position 0 starts from zero.
 #include "head_scan.h"
@@ -123,7 +123,7 @@ head_scan_chunk_kernel(const HeadScanArgs<T> a) {
           }
           if (a.silu_in) {
 #pragma unroll
-            for (int e = 0; e < 4; ++e) { qv[e] = silu_f(qv[e]); kv[e] = silu_f(kv[e]); }
+            for (int e = 0; e < 4; ++e) { qv[e] = silu_stored<T>(qv[e]); kv[e] = silu_stored<T>(kv[e]); }
           }
           if (DELTA) {
 #pragma unroll
@@ -349,16 +349,24 @@ hipError_t sm_head_scan_chunk(int dt, int delta, const void* q, long long ldq, c
     return hipErrorInvalidValue;
   const int vec = Dk % 4 == 0 && ldq % 4 == 0 && ldk % 4 == 0 && (uintptr_t)q % 16 == 0 &&
                   (uintptr_t)k % 16 == 0;
+#define ARGS(T)                                                                               \
+  HeadScanArgs<T> a{(const T*)q, ldq, (const T*)k, ldk, (const T*)v, ldv, (const T*)al, lda,  \
+                    (const T*)bl, ldb, A_log, dt_bias, log_decay, skip, state, out, cu, slot, \
+                    start, H, rep, Dk, Dv, silu_in, vec, key_eps, q_scale}
+  if (dt == kBF16) {
+    ARGS(bf16);
+    return head_scan_chunk16(a, delta != 0, n_seg, st);
+  }
 #define CALL(T)                                                                                 \
   {                                                                                             \
-    HeadScanArgs<T> a{(const T*)q, ldq, (const T*)k, ldk, (const T*)v, ldv, (const T*)al, lda,  \
-                      (const T*)bl, ldb, A_log, dt_bias, log_decay, skip, state, out, cu, slot, \
-                      start, H, rep, Dk, Dv, silu_in, vec, key_eps, q_scale};                   \
+    ARGS(T);                                                                                    \
     return delta ? launch_chunk<T, true>(a, n_seg, st) : launch_chunk<T, false>(a, n_seg, st);  \
   }
-  SM_DISPATCH(dt, CALL)
+  if (dt == kF32) CALL(float)
+  if (dt == kF16) CALL(fp16)
+  return hipErrorInvalidValue;
 #undef CALL
-  return hipSuccess;
+#undef ARGS
 }
 
 }  // extern "C"

@@ -70,7 +70,7 @@ __global__ void __launch_bounds__(256) head_scan_step_kernel(const HeadScanArgs<
       const int qc = (hd / a.rep) * Dk + tid;
       qv = to_f32(a.q[r * a.ldq + qc]);
       kv = to_f32(a.k[r * a.ldk + qc]);
-      if (a.silu_in) { qv = silu_f(qv); kv = silu_f(kv); }
+      if (a.silu_in) { qv = silu_stored<T>(qv); kv = silu_stored<T>(kv); }
     }
     float x[V], o[V];
 #pragma unroll
@@ -208,6 +208,34 @@ __global__ void __launch_bounds__(64) short_conv_kernel(const ConvArgs<T> a) {
   }
   float win[K > 0 ? K : 1][V];                       // win[d - 1]: the input d positions back
   const int t0 = blockIdx.y * kStrip, t1 = min(a.rows, t0 + kStrip);
+  // a whole strip of one segment: all its rows and the taps before them are loaded at once
+  if (t1 - t0 == kStrip && a.row_seg[t0] == a.row_seg[t1 - 1]) {
+    const int sg = a.row_seg[t0], local = t0 - a.cu[sg], p0 = a.start[sg];
+    float x[kStrip + K][V];
+#pragma unroll
+    for (int i = 0; i < kStrip; ++i) load_v<T, V>(a.x + (long long)(t0 + i) * a.ldx + c, x[K + i]);
+#pragma unroll
+    for (int d = 1; d <= K; ++d) {
+#pragma unroll
+      for (int j = 0; j < V; ++j) x[K - d][j] = 0.f;
+      const int src = local - d;
+      if (src >= 0) load_v<T, V>(a.x + (long long)(t0 - d) * a.ldx + c, x[K - d]);
+      else if (p0 + src >= 0) load_v<T, V>(a.tail + ((long long)a.slot[sg] * K + (K + src)) * a.C + c, x[K - d]);
+    }
+#pragma unroll
+    for (int i = 0; i < kStrip; ++i) {
+      float o[V];
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        float acc = wv[j][K] * x[K + i][j] + bv[j];
+#pragma unroll
+        for (int d = 1; d <= K; ++d) acc += wv[j][K - d] * x[K + i - d][j];
+        o[j] = silu_f(acc);
+      }
+      store_v<T, V>(a.out + (long long)(t0 + i) * a.C + c, o);
+    }
+    return;
+  }
   int cur = -1;
   for (int t = t0; t < t1; ++t) {
     const int sg = a.row_seg[t];

@@ -128,12 +128,14 @@ gated_rms_kernel(const float* __restrict__ x, const T* __restrict__ g, long long
         }
       }
     }
-    ss = wave_sum(ss);
-    if (lane == 0) s_part[wv] = ss;
-    __syncthreads();
-    if (on) {
-      float tot = 0.f;
+    float tot = wave_sum(ss);
+    if (wpg > 1) {                             // (uniform) waves sharing a group exchange their sums
+      if (lane == 0) s_part[wv] = tot;
+      __syncthreads();
+      tot = 0.f;
       for (int k = 0; k < wpg; ++k) tot += s_part[slot * wpg + k];
+    }
+    if (on) {
       const float inv = 1.f / sqrtf(tot / (float)gs + eps);
       for (int c = (sub * 64 + lane) * V; c < gs; c += wpg * 64 * V) {   // its own entries again
         const int col = gi * gs + c;
@@ -151,7 +153,7 @@ gated_rms_kernel(const float* __restrict__ x, const T* __restrict__ g, long long
         else orow[col] = from_f32<T>(v[0]);
       }
     }
-    __syncthreads();
+    if (wpg > 1) __syncthreads();
   }
 }
 

@@ -214,15 +214,15 @@ def min_gru_scan(zxg: torch.Tensor, b_z: torch.Tensor, b_x: torch.Tensor, state:
 # l = -exp(A_log) dt (the delta rule uses dt in the decay only).  The delta rule first makes q and k
 # unit vectors, x / sqrt(sum x^2 + key_eps), and multiplies q by ``q_scale``.  Decays, step sizes,
 # unit vectors and the state are fp32; the read-out is returned in fp32.
-# (HIP: ``csrc/seqmix/head_scan_chunk.hip`` for prompt portions, ``head_scan_step.hip`` for decoded
-# rows.)
+# (HIP: ``csrc/seqmix/head_scan_chunk.hip`` and, for bf16, ``head_scan_chunk16.hip`` for prompt
+# portions, ``head_scan_step.hip`` for decoded rows.)
 def head_scan_ref(q, k, v, state, seg: SegBatch, H, rep, Dk, Dv, decay, beta=None, skip=None,
                   silu_in=False, key_eps=0.0, q_scale=1.0):
     T = q.shape[0]
     act = F.silu if silu_in else (lambda t: t)
     hg = torch.arange(H, device=q.device) // rep
-    q_ = act(q.float().reshape(T, H // rep, Dk))
-    k_ = act(k.float().reshape(T, H // rep, Dk))
+    q_ = act(q.float().reshape(T, H // rep, Dk)).to(q.dtype).float()
+    k_ = act(k.float().reshape(T, H // rep, Dk)).to(k.dtype).float()
     v_ = act(v.float().reshape(T, H, Dv))
     if beta is not None:
         q_ = q_ / torch.sqrt((q_ * q_).sum(-1, keepdim=True) + key_eps) * q_scale
@@ -264,7 +264,7 @@ def head_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Te
     stride (slices of wider buffers are fine); ``state`` [slots, H, Dk, Dv] fp32 moves on.  ``decay``:
     an fp32 tensor [H] of constant log decays, or (logits [T, H], A_log [H], dt_bias [H]).  ``beta``
     [T, H] (write-strength logits) selects the delta rule, without ``skip``.  ``silu_in``: q, k and v
-    pass through silu as they are read.  Returns the read-outs [T, H * Dv] in fp32."""
+    pass through silu as they are read (q and k rounded to their dtype again).  Returns the read-outs [T, H * Dv] in fp32."""
     from ._seqmix import DT, call, use_seqmix
 
     if H % rep:
