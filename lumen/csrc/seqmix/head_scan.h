@@ -42,6 +42,13 @@ __device__ __forceinline__ void head_decay(const HeadScanArgs<T>& s, long long r
   ld = fmaxf(ld, -1e4f);
 }
 
+// silu of a value that is stored as T next: 16-bit types take the hardware exponential and
+// reciprocal, whose last-place error disappears in the rounding
+template <typename T> __device__ __forceinline__ float silu_as(float x) {
+  return x * __builtin_amdgcn_rcpf(1.f + __expf(-x));
+}
+template <> __device__ __forceinline__ float silu_as<float>(float x) { return silu_f(x); }
+
 // silu of a stored q or k element, rounded to its type again: what a projection with an activation
 // stores, so that every kernel multiplies the same values
 template <typename T> __device__ __forceinline__ float silu_stored(float x) {

@@ -14,10 +14,11 @@
 // (three where both sides are split) keep ~16 mantissa bits; sums are fp32.  The state itself
 // stays fp32 in accumulator registers, a wave holding [Dk x 32 value columns].
 //
-// A workgroup is NW column waves and ONE producer wave, and two LDS buffers: while the column waves
-// run chunk n, the producer builds chunk n + 1 -- q, k and k transposed from registers it loaded
-// one chunk earlier, decays, Q K^T, K K^T, the triangular inverse -- and starts loading chunk n + 2.
-// One barrier per chunk.
+// A workgroup is NW column waves and TWO producer waves, and two LDS buffers: while the column waves
+// run chunk n, the producers build chunk n + 1 in two phases with a barrier after each.  First one
+// stores q and the decays, the other k and k transposed, from registers they loaded one chunk
+// earlier, and both start loading chunk n + 2 (meanwhile the column waves take Q S_0 and K S_0);
+// then one forms G . Q K^T and the other the triangular inverse (meanwhile: U, O and the state).
 //
 // 32x32x16 products: accumulator register r of lane half hi is row 8 (r >> 2) + 4 hi + (r & 3); the
 // registers 8s .. 8s+7 therefore hold inner indices {16s + 4hi + 0..3, 16s + 8 + 4hi + 0..3} and are
@@ -111,14 +112,14 @@ __device__ __forceinline__ float diagonal(const f32x16& x, int c, int hi) {
 }
 
 template <int KT, int NW, bool DELTA>
-__global__ void __launch_bounds__(64 * (NW + 1))
+__global__ void __launch_bounds__(64 * (NW + 2))
 head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
   constexpr int DKP = 32 * KT, LK = DKP + 8, NV = DKP / 8;
   constexpr int NI = (DKP + 63) / 64;          // items per producer lane and matrix
   using Buf = ChunkBuf<DKP, DELTA>;
   __shared__ Buf s_buf[2];
-  __shared__ __align__(16) double s_L[kC];     // the producer's: log-decay sums, unit factors, beta
-  __shared__ __align__(16) float s_fk[kC], s_be[kC];
+  __shared__ __align__(16) double s_L[kC];     // the producers': log-decay sums, unit factors
+  __shared__ __align__(16) float s_fk[2][kC];
   const int sg = blockIdx.x, hd = blockIdx.y;
   const int r0 = a.cu[sg], len = a.cu[sg + 1] - r0;
   if (len <= 0) return;
@@ -129,19 +130,21 @@ head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
 
   // Rows past the segment's end are read as its last row: their step size (or beta) is zero, so
   // they add nothing to the state, and their read-outs are not stored.
-  if (w == NW) {
-    // ---------------- the producer wave ----------------
-    Item iq[NI], ik[NI];
+  if (w >= NW) {
+    // ---------------- the producer waves ----------------
+    const bool is_k = w > NW;
+    const bf16* base = is_k ? a.k : a.q;
+    const long long ldr = is_k ? a.ldk : a.ldq;
+    Item it[NI];
     float ra = 0.f, rb = 0.f;                  // the token's decay and write-strength logits
-    auto fetch_rows = [&](const bf16* base, long long ld, int t0, Item (&it)[NI])
-        __attribute__((always_inline)) {
+    auto fetch = [&](int t0) __attribute__((always_inline)) {
 #pragma unroll
       for (int x = 0; x < NI; ++x) {
         const int item = lane + 64 * x, kq = (item / NV) & 7, d = 8 * (item % NV);
 #pragma unroll
         for (int y = 0; y < 4; ++y) {
           const int i = min(t0 + 4 * kq + y, len - 1);
-          const bf16* p = base + (long long)(r0 + i) * ld + qcol + d;
+          const bf16* p = base + (long long)(r0 + i) * ldr + qcol + d;
           uint4 v = make_uint4(0, 0, 0, 0);
           if (d < Dk) {
             if (a.vec) {
@@ -158,21 +161,21 @@ head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
           it[x].r[y] = v;
         }
       }
-    };
-    auto fetch = [&](int t0) __attribute__((always_inline)) {
-      fetch_rows(a.q, a.ldq, t0, iq);
-      fetch_rows(a.k, a.ldk, t0, ik);
-      const long long i = r0 + min(t0 + c, len - 1);
-      if (a.a != nullptr) ra = to_f32(a.a[i * a.lda + hd]);
-      if (DELTA) rb = to_f32(a.b[i * a.ldb + hd]);
+      if (!is_k) {
+        const long long i = r0 + min(t0 + c, len - 1);
+        if (a.a != nullptr) ra = to_f32(a.a[i * a.lda + hd]);
+        if (DELTA) rb = to_f32(a.b[i * a.ldb + hd]);
+      }
     };
     const float dtb = a.a != nullptr ? a.dt_bias[hd] : 0.f;
     const float eA = a.a != nullptr ? expf(a.A_log[hd]) : 0.f;
     const float ldc = a.a != nullptr ? 0.f : a.log_decay[hd];
 
-    auto put_rows = [&](Item (&it)[NI], bf16* dst, bf16* kt, auto is_k)
-        __attribute__((always_inline)) {
-      constexpr bool IS_K = decltype(is_k)::value;
+    double L = 0.0, Lc = 0.0;                  // (the q wave) the lane's log-decay sum, the chunk's
+
+    // phase 1: rows into LDS, decays
+    auto rows = [&](int t0, Buf& B) __attribute__((always_inline)) {
+      bf16* dst = is_k ? B.k : B.q;
 #pragma unroll
       for (int x = 0; x < NI; ++x) {
         const int item = lane + 64 * x, kq = item / NV, part = item % NV;
@@ -191,14 +194,14 @@ head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
             *reinterpret_cast<uint2*>(row) = make_uint2(it[x].r[y].x, it[x].r[y].y);
             *reinterpret_cast<uint2*>(row + 8) = make_uint2(it[x].r[y].z, it[x].r[y].w);
           }
-          if (IS_K) {                          // transposed: 4 tokens of each of the 8 channels
+          if (is_k) {                          // transposed: 4 tokens of each of the 8 channels
             const unsigned e0[4] = {it[x].r[0].x, it[x].r[0].y, it[x].r[0].z, it[x].r[0].w};
             const unsigned e1[4] = {it[x].r[1].x, it[x].r[1].y, it[x].r[1].z, it[x].r[1].w};
             const unsigned e2[4] = {it[x].r[2].x, it[x].r[2].y, it[x].r[2].z, it[x].r[2].w};
             const unsigned e3[4] = {it[x].r[3].x, it[x].r[3].y, it[x].r[3].z, it[x].r[3].w};
             // 16-byte unit of the row (swapped by the channel group: lanes spread over banks)
             const int unit = (2 * (kq >> 2) + (kq & 1)) ^ (part & 3);
-            bf16* t = kt + 8 * part * LT + 8 * unit + 4 * ((kq >> 1) & 1);
+            bf16* t = B.kt + 8 * part * LT + 8 * unit + 4 * ((kq >> 1) & 1);
 #pragma unroll
             for (int z = 0; z < 4; ++z) {
               *reinterpret_cast<uint2*>(t + 2 * z * LT) =
@@ -209,34 +212,32 @@ head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
           }
         }
       }
-    };
-    auto build = [&](int t0, Buf& B) __attribute__((always_inline)) {
-      const int n = min(kC, len - t0);
-      put_rows(iq, B.q, B.kt, std::false_type{});
-      put_rows(ik, B.k, B.kt, std::true_type{});
-      // decays: lane c (both halves alike) is token c; tokens past the end add nothing
-      float ld = 0.f, wt = 0.f, dt = 1.f;
-      if (a.a != nullptr) {
-        dt = softplus_f(ra + dtb);
-        ld = -eA * dt;
-      } else {
-        ld = ldc;
-      }
-      wt = DELTA ? sigmoid_f(rb) : dt;
-      ld = c < n ? fmaxf(ld, -1e4f) : 0.f;
-      wt = c < n ? wt : 0.f;
-      if (!DELTA && t0 + kC < len) fetch(t0 + kC);     // the next chunk's rows travel meanwhile
-      double L = (double)ld;
+      if (!is_k) {
+        // lane c (both halves alike) is token c; tokens past the end add nothing
+        const bool live = t0 + c < len;
+        float ld = ldc, dt = 1.f;
+        if (a.a != nullptr) {
+          dt = softplus_f(ra + dtb);
+          ld = -eA * dt;
+        }
+        const float wt = DELTA ? sigmoid_f(rb) : dt;
+        L = live ? (double)fmaxf(ld, -1e4f) : 0.0;
 #pragma unroll
-      for (int m = 1; m < 32; m <<= 1) {
-        const double o = __shfl_up(L, m, 32);
-        if (c >= m) L += o;
+        for (int m = 1; m < 32; m <<= 1) {
+          const double o = __shfl_up(L, m, 32);
+          if (c >= m) L += o;
+        }
+        Lc = __shfl(L, 31, 32);
+        if (hi == 0) {
+          s_L[c] = L;
+          B.w[c] = live ? wt : 0.f;
+        }
       }
-      const double Lc = __shfl(L, 31, 32);
-      if (hi == 0) s_L[c] = L;
-      if (DELTA && hi == 0) s_be[c] = wt;
-      wave_lds_fence();
-      // P^T = K Q^T (lane: query, registers: keys) and K K^T, Q Q^T (unit lengths: their diagonals)
+      if (t0 + kC < len) fetch(t0 + kC);       // the next chunk's rows travel meanwhile
+    };
+
+    // phase 2: P^T = K Q^T (lane: query, registers: keys) times G, and the chunk's factors
+    auto weights = [&](Buf& B) __attribute__((always_inline)) {
       f32x16 P, A, Q;
 #pragma unroll
       for (int r = 0; r < 16; ++r) { P[r] = 0.f; A[r] = 0.f; Q[r] = 0.f; }
@@ -245,7 +246,7 @@ head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
         const uint4 kv = *reinterpret_cast<const uint4*>(B.k + c * LK + 16 * s + 8 * hi);
         const uint4 qv = *reinterpret_cast<const uint4*>(B.q + c * LK + 16 * s + 8 * hi);
         P = mma(kv, qv, P);
-        if (DELTA) {
+        if (DELTA) {                           // unit lengths: the diagonals of K K^T and Q Q^T
           A = mma(kv, kv, A);
           Q = mma(qv, qv, Q);
         }
@@ -254,109 +255,135 @@ head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
       if (DELTA) {
         fqc = a.q_scale / sqrtf(diagonal(Q, c, hi) + a.key_eps);
         fkc = 1.f / sqrtf(diagonal(A, c, hi) + a.key_eps);
-        if (hi == 0) s_fk[c] = fkc;
+        if (hi == 0) s_fk[0][c] = fkc;
         wave_lds_fence();
-        if (t0 + kC < len) fetch(t0 + kC);     // (Q Q^T's registers are free again)
       }
       if (hi == 0) {
         const float g = expf((float)L);
         B.gq[c] = g * fqc;
         B.gk[c] = g * fkc;
-        B.w[c] = wt;
         B.ek[c] = expf((float)(Lc - L)) * fkc;
         if (c == 0) B.gc = expf((float)Lc);
       }
-      // registers: tokens j = 8 g + 4 hi + e; the lane's own token is c
-      float* sA = reinterpret_cast<float*>(B.p[0]);    // the inverse's scratch: before p is written
-      static_assert(!DELTA || sizeof(float) * kC * LA <= sizeof(B.p), "scratch fits");
+#pragma unroll
+      for (int g = 0; g < 4; ++g) {
+        const int j0 = 8 * g + 4 * hi;         // registers 4g + e: token j0 + e
+        const double2 La = *reinterpret_cast<const double2*>(&s_L[j0]);
+        const double2 Lb = *reinterpret_cast<const double2*>(&s_L[j0 + 2]);
+        const float d[4] = {(float)(L - La.x), (float)(L - La.y), (float)(L - Lb.x),
+                            (float)(L - Lb.y)};
+        float fk[4] = {1.f, 1.f, 1.f, 1.f}, z[4];
+        if (DELTA) load4<float>(&s_fk[0][j0], fk);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float v = P[4 * g + e] * (fqc * fk[e]) * __expf(fminf(d[e], 0.f));
+          z[e] = j0 + e <= c ? v : 0.f;
+        }
+        const int at = c * LT + place(j0);
+        put4(&B.p[0][at], &B.p[1][at], z[0], z[1], z[2], z[3]);
+      }
+    };
+
+    // phase 2, delta rule: T = (I + A)^-1
+    auto inverse = [&](Buf& B) __attribute__((always_inline)) {
+      f32x16 A;
+#pragma unroll
+      for (int r = 0; r < 16; ++r) A[r] = 0.f;
+#pragma unroll
+      for (int s = 0; s < 2 * KT; ++s) {
+        const uint4 kv = *reinterpret_cast<const uint4*>(B.k + c * LK + 16 * s + 8 * hi);
+        A = mma(kv, kv, A);
+      }
+      const float fkc = 1.f / sqrtf(diagonal(A, c, hi) + a.key_eps);
+      if (hi == 0) s_fk[1][c] = fkc;
+      wave_lds_fence();
+      // scratch, transposed: row c, entry j = A[j][c] (j > c); it lies where T is written later
+      float* sA = reinterpret_cast<float*>(B.t[0]);
+      static_assert(!DELTA || sizeof(float) * kC * LA <= sizeof(B.t), "scratch fits");
+      const double Lo = s_L[c];
 #pragma unroll
       for (int g = 0; g < 4; ++g) {
         const int j0 = 8 * g + 4 * hi;
         const double2 La = *reinterpret_cast<const double2*>(&s_L[j0]);
         const double2 Lb = *reinterpret_cast<const double2*>(&s_L[j0 + 2]);
-        const float d[4] = {(float)(L - La.x), (float)(L - La.y), (float)(L - Lb.x),
-                            (float)(L - Lb.y)};
-        float fk[4] = {1.f, 1.f, 1.f, 1.f};
-        if (DELTA) {
-          float be[4], x[4];
-          load4<float>(&s_fk[j0], fk);
-          load4<float>(&s_be[j0], be);
-          // transposed scratch: row c, entry j = A[j][c] (j > c)
+        const float d[4] = {(float)(La.x - Lo), (float)(La.y - Lo), (float)(Lb.x - Lo),
+                            (float)(Lb.y - Lo)};
+        float fk[4], be[4], x[4];
+        load4<float>(&s_fk[1][j0], fk);
+        load4<float>(&B.w[j0], be);
 #pragma unroll
-          for (int e = 0; e < 4; ++e)
-            x[e] = j0 + e > c ? A[4 * g + e] * (fk[e] * fkc) * (be[e] * __expf(fminf(-d[e], 0.f))) : 0.f;
-          store4<float>(&sA[c * LA + j0], x);
+        for (int e = 0; e < 4; ++e)
+          x[e] = j0 + e > c ? A[4 * g + e] * (fk[e] * fkc) * (be[e] * __expf(fminf(d[e], 0.f))) : 0.f;
+        store4<float>(&sA[c * LA + j0], x);
+      }
+      wave_lds_fence();
+      // the diagonal 16x16 blocks by back substitution along a row,
+      // T[i][j] = [i = j] - sum_{k > j} T[i][k] A[k][j], a lane per row i ...
+      const int b0 = lane & 16, ii = lane & 15, lr = lane & 15, lg = lane >> 4;
+      float t[16];
+#pragma unroll
+      for (int j = 15; j >= 0; --j) {
+        float acc = 0.f;
+#pragma unroll
+        for (int k4 = 0; k4 < 16; k4 += 4) {
+          if (k4 + 3 > j) {
+            const float4 x = *reinterpret_cast<const float4*>(&sA[(b0 + j) * LA + b0 + k4]);
+            if (k4 > j) acc += x.x * t[k4];
+            if (k4 + 1 > j) acc += x.y * t[k4 + 1];
+            if (k4 + 2 > j) acc += x.z * t[k4 + 2];
+            acc += x.w * t[k4 + 3];
+          }
         }
+        t[j] = j == ii ? 1.f : (j < ii ? -acc : 0.f);
+      }
+      wave_lds_fence();
+      if (lane < 32) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const float z = P[4 * g + e] * (fqc * fk[e]) * __expf(fminf(d[e], 0.f));
-          P[4 * g + e] = j0 + e <= c ? z : 0.f;
+        for (int j = 0; j < 16; j += 4)
+          *reinterpret_cast<float4*>(&sA[(b0 + ii) * LA + b0 + j]) =
+              make_float4(t[j], t[j + 1], t[j + 2], t[j + 3]);
+      }
+      wave_lds_fence();
+      // ... and the block below as -T11 (A10 T00); A10[r][k] lies at scratch [k][16 + r]
+      f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int m = 0; m < 4; ++m)
+        x = mma16f(sA[(4 * m + lg) * LA + 16 + lr], sA[(4 * m + lg) * LA + lr], x);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y = mma16f(sA[(16 + lr) * LA + 16 + 4 * lg + e], x[e], y);
+      wave_lds_fence();                        // scratch read: T may be written over it
+      bf16 *th = B.t[0], *tl = B.t[DELTA ? 1 : 0];
+      if (lane < 32) {
+#pragma unroll
+        for (int j = 0; j < 16; j += 4) {
+          const int at = (b0 + ii) * LT + place(b0 + j);
+          put4(th + at, tl + at, t[j], t[j + 1], t[j + 2], t[j + 3]);
+        }
+      } else if (lane < 48) {                  // the block above the diagonal
+#pragma unroll
+        for (int j = 16; j < 32; j += 4) {
+          const int at = ii * LT + place(j);
+          put4(th + at, tl + at, 0.f, 0.f, 0.f, 0.f);
         }
       }
-      if (DELTA) {
-        wave_lds_fence();
-        // T = (I + A)^-1: the diagonal 16x16 blocks by back substitution along a row,
-        // T[i][j] = [i = j] - sum_{k > j} T[i][k] A[k][j], a lane per row i ...
-        const int b0 = lane & 16, ii = lane & 15, lr = lane & 15, lg = lane >> 4;
-        float t[16];
 #pragma unroll
-        for (int j = 15; j >= 0; --j) {
-          float acc = 0.f;
-#pragma unroll
-          for (int k4 = 0; k4 < 16; k4 += 4) {
-            if (k4 + 3 > j) {
-              const float4 x = *reinterpret_cast<const float4*>(&sA[(b0 + j) * LA + b0 + k4]);
-              if (k4 > j) acc += x.x * t[k4];
-              if (k4 + 1 > j) acc += x.y * t[k4 + 1];
-              if (k4 + 2 > j) acc += x.z * t[k4 + 2];
-              acc += x.w * t[k4 + 3];
-            }
-          }
-          t[j] = j == ii ? 1.f : (j < ii ? -acc : 0.f);
-        }
-        wave_lds_fence();
-        if (lane < 32) {
-#pragma unroll
-          for (int j = 0; j < 16; j += 4) {
-            *reinterpret_cast<float4*>(&sA[(b0 + ii) * LA + b0 + j]) =
-                make_float4(t[j], t[j + 1], t[j + 2], t[j + 3]);
-            const int at = (b0 + ii) * LT + place(b0 + j);
-            put4(&B.t[0][at], &B.t[DELTA ? 1 : 0][at], t[j], t[j + 1], t[j + 2], t[j + 3]);
-          }
-        } else if (lane < 48) {                // the block above the diagonal
-#pragma unroll
-          for (int j = 16; j < 32; j += 4) {
-            const int at = ii * LT + place(j);
-            put4(&B.t[0][at], &B.t[DELTA ? 1 : 0][at], 0.f, 0.f, 0.f, 0.f);
-          }
-        }
-        wave_lds_fence();
-        // ... and the block below as -T11 (A10 T00); A10[r][k] lies at scratch [k][16 + r]
-        f32x4 x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int m = 0; m < 4; ++m)
-          x = mma16f(sA[(4 * m + lg) * LA + 16 + lr], sA[(4 * m + lg) * LA + lr], x);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) y = mma16f(sA[(16 + lr) * LA + 16 + 4 * lg + e], x[e], y);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const int at = (16 + 4 * lg + e) * LT + place(lr);
-          const bf16 h = __float2bfloat16(-y[e]);
-          B.t[0][at] = h;
-          B.t[DELTA ? 1 : 0][at] = __float2bfloat16(-y[e] - __bfloat162float(h));
-        }
-        wave_lds_fence();                      // scratch read: p may be written
-      }
-#pragma unroll
-      for (int g = 0; g < 4; ++g) {
-        const int at = c * LT + place(8 * g + 4 * hi);
-        put4(&B.p[0][at], &B.p[1][at], P[4 * g], P[4 * g + 1], P[4 * g + 2], P[4 * g + 3]);
+      for (int e = 0; e < 4; ++e) {
+        const int at = (16 + 4 * lg + e) * LT + place(lr);
+        const bf16 h = __float2bfloat16(-y[e]);
+        th[at] = h;
+        tl[at] = __float2bfloat16(-y[e] - __bfloat162float(h));
       }
     };
 
     fetch(0);
     for (int n = 0; n <= chunks; ++n) {        // chunk n is built while the others run chunk n - 1
-      if (n < chunks) build(n * kC, s_buf[n & 1]);
+      Buf& B = s_buf[n & 1];
+      if (n < chunks) rows(n * kC, B);
+      __syncthreads();
+      if (n < chunks) {
+        if (!is_k) weights(B);
+        else if (DELTA) inverse(B);
+      }
       __syncthreads();
     }
     return;
@@ -389,6 +416,7 @@ head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
   };
   fetch_v(0);
   __syncthreads();
+  __syncthreads();
   for (int ch = 0; ch < chunks; ++ch) {
     const Buf& B = s_buf[ch & 1];
     const int t0 = ch * kC, n = min(kC, len - t0);
@@ -419,6 +447,7 @@ head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
           U = mma(kv, l, U);
         }
       }
+    __syncthreads();
     // the chunk matrices times a split right operand
     auto apply = [&](const bf16* mh, const bf16* ml, const f32x16& x, f32x16 acc) __attribute__((always_inline)) {
 #pragma unroll
@@ -509,15 +538,18 @@ head_scan_chunk16_kernel(const HeadScanArgs<bf16> a) {
 
 template <bool DELTA>
 hipError_t launch(const HeadScanArgs<bf16>& a, int n_seg, hipStream_t st) {
-  const int cb = (a.Dv + 31) / 32;                   // 32-column blocks
+  // 32-column blocks; a grid that leaves half the CUs idle is cut finer (each column block's result
+  // is the same whichever workgroup computes it)
+  const int cb = (a.Dv + 31) / 32;
+  const bool fine = cb > 2 && (long long)n_seg * a.H * ((cb + 3) / 4) <= 128;
 #define GO(KT, NW)                                                             \
   head_scan_chunk16_kernel<KT, NW, DELTA>                                      \
-      <<<dim3(n_seg, a.H, (cb + NW - 1) / NW), 64 * (NW + 1), 0, st>>>(a)
-#define GO_K(KT)                 \
-  if (cb == 1) GO(KT, 1);        \
-  else if (cb == 2) GO(KT, 2);   \
-  else if (cb == 3 || KT == 8) GO(KT, 3);   /* 256 state rows: four waves' registers */ \
-  else GO(KT, (KT == 8 ? 3 : 4))
+      <<<dim3(n_seg, a.H, (cb + NW - 1) / NW), 64 * (NW + 2), 0, st>>>(a)
+#define GO_K(KT)                                                               \
+  if (cb == 1) GO(KT, 1);                                                      \
+  else if (cb == 2 || fine) GO(KT, 2);                                         \
+  else if (cb == 3) GO(KT, (KT == 8 ? 2 : 3));                                 \
+  else GO(KT, (KT == 8 ? 2 : 4))   /* 256 state rows: two column waves' registers */
   if (a.Dk <= 32) { GO_K(1); }
   else if (a.Dk <= 64) { GO_K(2); }
   else if (a.Dk <= 128) { GO_K(4); }

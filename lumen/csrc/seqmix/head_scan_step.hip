@@ -209,32 +209,35 @@ __global__ void __launch_bounds__(64) short_conv_kernel(const ConvArgs<T> a) {
   float win[K > 0 ? K : 1][V];                       // win[d - 1]: the input d positions back
   const int t0 = blockIdx.y * kStrip, t1 = min(a.rows, t0 + kStrip);
   // a whole strip of one segment: all its rows and the taps before them are loaded at once
-  if (t1 - t0 == kStrip && a.row_seg[t0] == a.row_seg[t1 - 1]) {
-    const int sg = a.row_seg[t0], local = t0 - a.cu[sg], p0 = a.start[sg];
+  if (t1 - t0 == kStrip) {
     float x[kStrip + K][V];
 #pragma unroll
     for (int i = 0; i < kStrip; ++i) load_v<T, V>(a.x + (long long)(t0 + i) * a.ldx + c, x[K + i]);
+    const int sg = a.row_seg[t0];
+    if (sg == a.row_seg[t1 - 1]) {
+      const int local = t0 - a.cu[sg], p0 = a.start[sg];
 #pragma unroll
-    for (int d = 1; d <= K; ++d) {
+      for (int d = 1; d <= K; ++d) {
 #pragma unroll
-      for (int j = 0; j < V; ++j) x[K - d][j] = 0.f;
-      const int src = local - d;
-      if (src >= 0) load_v<T, V>(a.x + (long long)(t0 - d) * a.ldx + c, x[K - d]);
-      else if (p0 + src >= 0) load_v<T, V>(a.tail + ((long long)a.slot[sg] * K + (K + src)) * a.C + c, x[K - d]);
-    }
-#pragma unroll
-    for (int i = 0; i < kStrip; ++i) {
-      float o[V];
-#pragma unroll
-      for (int j = 0; j < V; ++j) {
-        float acc = wv[j][K] * x[K + i][j] + bv[j];
-#pragma unroll
-        for (int d = 1; d <= K; ++d) acc += wv[j][K - d] * x[K + i - d][j];
-        o[j] = silu_f(acc);
+        for (int j = 0; j < V; ++j) x[K - d][j] = 0.f;
+        const int src = local - d;
+        if (src >= 0) load_v<T, V>(a.x + (long long)(t0 - d) * a.ldx + c, x[K - d]);
+        else if (p0 + src >= 0) load_v<T, V>(a.tail + ((long long)a.slot[sg] * K + (K + src)) * a.C + c, x[K - d]);
       }
-      store_v<T, V>(a.out + (long long)(t0 + i) * a.C + c, o);
+#pragma unroll
+      for (int i = 0; i < kStrip; ++i) {
+        float o[V];
+#pragma unroll
+        for (int j = 0; j < V; ++j) {
+          float acc = wv[j][K] * x[K + i][j] + bv[j];
+#pragma unroll
+          for (int d = 1; d <= K; ++d) acc += wv[j][K - d] * x[K + i - d][j];
+          o[j] = silu_as<T>(acc);
+        }
+        store_v<T, V>(a.out + (long long)(t0 + i) * a.C + c, o);
+      }
+      return;
     }
-    return;
   }
   int cur = -1;
   for (int t = t0; t < t1; ++t) {
@@ -261,7 +264,7 @@ __global__ void __launch_bounds__(64) short_conv_kernel(const ConvArgs<T> a) {
       float acc = wv[j][K] * h[j] + bv[j];
 #pragma unroll
       for (int d = 1; d <= K; ++d) acc += wv[j][K - d] * win[d - 1][j];
-      o[j] = silu_f(acc);
+      o[j] = silu_as<T>(acc);
     }
     store_v<T, V>(a.out + (long long)t * a.C + c, o);
 #pragma unroll
@@ -292,7 +295,7 @@ __global__ void __launch_bounds__(256) short_conv_any_kernel(const ConvArgs<T> a
       else if (p0 + src >= 0) h = to_f32(a.tail[((long long)a.slot[sg] * K + (K + src)) * a.C + c]);
       acc += a.w[(long long)c * a.taps + (K - d)] * h;
     }
-    a.out[(long long)t * a.C + c] = from_f32<T>(silu_f(acc));
+    a.out[(long long)t * a.C + c] = from_f32<T>(silu_as<T>(acc));
   }
 }
 
@@ -317,7 +320,7 @@ __global__ void __launch_bounds__(256) conv_tail_kernel(const ConvArgs<T> a) {
 #pragma unroll
     for (int k = 0; k < kMaxTaps; ++k)
       if (k < K) acc += w[k] * to_f32(old[k]);
-    a.out[(long long)r0 * a.C + c] = from_f32<T>(silu_f(acc));
+    a.out[(long long)r0 * a.C + c] = from_f32<T>(silu_as<T>(acc));
 #pragma unroll
     for (int k = 0; k < kMaxTaps - 1; ++k)
       if (k < K) tp[(long long)k * a.C] = k == K - 1 ? h : old[k + 1];

@@ -166,6 +166,7 @@ constexpr int kMaxHead = 512;
 // one workgroup per row.  The row's dims / 2 sines and cosines are computed once, in LDS, for all
 // heads; a subgroup of SG lanes (a power of two, 4 entries per lane) owns a head, so that a
 // wave works on 64 / SG heads at a time; the pair partner dims / 2 entries away is a lane exchange.
+// A step with few rows deals a row's heads out to several workgroups (grid y).
 template <typename T>
 __global__ void __launch_bounds__(kThreads) head_norm_rotary_v4(const HeadArgs<T> a, int SG) {
   __shared__ float s_cs[kMaxHead / 2], s_sn[kMaxHead / 2];
@@ -179,7 +180,7 @@ __global__ void __launch_bounds__(kThreads) head_norm_rotary_v4(const HeadArgs<T
   const int sub = threadIdx.x / SG, nsub = kThreads / SG, sl = lane & (SG - 1), sb = lane & ~(SG - 1);
   const int items = a.H + 2 * a.G;
   // every lane of a wave runs the same number of rounds: the exchanges below need all of them
-  for (int i0 = 0; i0 < items; i0 += nsub) {
+  for (int i0 = blockIdx.y * nsub; i0 < items; i0 += gridDim.y * nsub) {
     const int item = i0 + sub;
     const bool live = item < items;
     const bool is_v = item >= a.H + a.G, is_q = item < a.H;
@@ -338,11 +339,13 @@ hipError_t sm_head_norm_rotary(int dt, void* z, long long ld, const float* wq, c
                    (uintptr_t)wq % 16 == 0 && (uintptr_t)wk % 16 == 0;
   int SG = 1;
   while (4 * SG < m) SG <<= 1;
+  const int rounds = (H + 2 * G + kThreads / SG - 1) / (kThreads / SG);
+  const dim3 grid(T, T <= 64 ? rounds : 1);
 #define CALL(TT)                                                                                \
   {                                                                                             \
     HeadArgs<TT> a{(TT*)z, ld, wq, wk, positions, slots, (TT*)kc, (TT*)vc, inv_freq, H, G, D,   \
                    Dv, dims, vnorm, eps};                                                       \
-    if (vec) head_norm_rotary_v4<TT><<<T, kThreads, 0, st>>>(a, SG);                            \
+    if (vec) head_norm_rotary_v4<TT><<<grid, kThreads, 0, st>>>(a, SG);                         \
     else head_norm_rotary_any<TT><<<T, kThreads, 0, st>>>(a);                                   \
   }
   SM_DISPATCH(dt, CALL)

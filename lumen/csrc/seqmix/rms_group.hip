@@ -87,8 +87,9 @@ group_rms_kernel(const TI* __restrict__ x, long long ldx, const float* __restric
   }
 }
 
-// the row (gated, when the gate comes first) stays in LDS between the two passes; groups are dealt
-// out to the waves as above
+// four or more groups: a wave per group, blockIdx.y naming the four a workgroup takes; fewer: one
+// workgroup per row as above.  The entries (gated, when the gate comes first) stay in LDS between the
+// two passes.
 template <typename T, bool VEC>
 __global__ void __launch_bounds__(256)
 gated_rms_kernel(const float* __restrict__ x, const T* __restrict__ g, long long ldg,
@@ -105,56 +106,87 @@ gated_rms_kernel(const float* __restrict__ x, const T* __restrict__ g, long long
   const T* gr = g + (long long)r * ldg;
   T* orow = out + (long long)r * W;
   constexpr int V = VEC ? 4 : 1;
-  for (int g0 = 0; g0 < groups; g0 += per_pass) {
-    const int gi = g0 + slot;
-    const bool on = gi < groups && slot < per_pass;
-    float ss = 0.f;
-    if (on) {
-      for (int c = (sub * 64 + lane) * V; c < gs; c += wpg * 64 * V) {
-        const int col = gi * gs + c;
-        float v[V], z[V];
-        if constexpr (VEC) load4<float>(xr + col, v);
-        else v[0] = xr[col];
-        if (gate_first) {
-          if constexpr (VEC) load4<T>(gr + col, z);
-          else z[0] = to_f32(gr[col]);
+  const int gi = blockIdx.y * per_pass + slot;
+  const bool on = gi < groups && slot < per_pass;
+  float ss = 0.f;
+  if (on) {
+    for (int c = (sub * 64 + lane) * V; c < gs; c += wpg * 64 * V) {
+      const int col = gi * gs + c;
+      float v[V], z[V];
+      if constexpr (VEC) load4<float>(xr + col, v);
+      else v[0] = xr[col];
+      if (gate_first) {
+        if constexpr (VEC) load4<T>(gr + col, z);
+        else z[0] = to_f32(gr[col]);
 #pragma unroll
-          for (int e = 0; e < V; ++e) v[e] *= sigmoid ? sigmoid_f(z[e]) : silu_f(z[e]);
-        }
+        for (int e = 0; e < V; ++e) v[e] *= sigmoid ? sigmoid_f(z[e]) : silu_f(z[e]);
+      }
 #pragma unroll
-        for (int e = 0; e < V; ++e) {
-          ss += v[e] * v[e];
-          s_row[col + e] = v[e];
-        }
+      for (int e = 0; e < V; ++e) {
+        ss += v[e] * v[e];
+        s_row[slot * gs + c + e] = v[e];
       }
     }
-    float tot = wave_sum(ss);
-    if (wpg > 1) {                             // (uniform) waves sharing a group exchange their sums
-      if (lane == 0) s_part[wv] = tot;
-      __syncthreads();
-      tot = 0.f;
-      for (int k = 0; k < wpg; ++k) tot += s_part[slot * wpg + k];
-    }
-    if (on) {
-      const float inv = 1.f / sqrtf(tot / (float)gs + eps);
-      for (int c = (sub * 64 + lane) * V; c < gs; c += wpg * 64 * V) {   // its own entries again
-        const int col = gi * gs + c;
-        const float* wp = w + (shared_w ? c : col);
-        float v[V], z[V];
-#pragma unroll
-        for (int e = 0; e < V; ++e) v[e] = s_row[col + e] * inv * wp[e];
-        if (!gate_first) {
-          if constexpr (VEC) load4<T>(gr + col, z);
-          else z[0] = to_f32(gr[col]);
-#pragma unroll
-          for (int e = 0; e < V; ++e) v[e] *= sigmoid ? sigmoid_f(z[e]) : silu_f(z[e]);
-        }
-        if constexpr (VEC) store4<T>(orow + col, v);
-        else orow[col] = from_f32<T>(v[0]);
-      }
-    }
-    if (wpg > 1) __syncthreads();
   }
+  float tot = wave_sum(ss);
+  if (wpg > 1) {                             // (uniform) waves sharing a group exchange their sums
+    if (lane == 0) s_part[wv] = tot;
+    __syncthreads();
+    tot = 0.f;
+    for (int k = 0; k < wpg; ++k) tot += s_part[slot * wpg + k];
+  }
+  if (on) {
+    const float inv = 1.f / sqrtf(tot / (float)gs + eps);
+    for (int c = (sub * 64 + lane) * V; c < gs; c += wpg * 64 * V) {   // its own entries again
+      const int col = gi * gs + c;
+      const float* wp = w + (shared_w ? c : col);
+      float v[V], z[V];
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] = s_row[slot * gs + c + e] * inv * wp[e];
+      if (!gate_first) {
+        if constexpr (VEC) load4<T>(gr + col, z);
+        else z[0] = to_f32(gr[col]);
+#pragma unroll
+        for (int e = 0; e < V; ++e) v[e] *= sigmoid ? sigmoid_f(z[e]) : silu_f(z[e]);
+      }
+      if constexpr (VEC) store4<T>(orow + col, v);
+      else orow[col] = from_f32<T>(v[0]);
+    }
+  }
+}
+
+// groups of at most 256 entries (heads): SG lanes of 4 entries each own a (row, group), in registers
+template <typename T>
+__global__ void __launch_bounds__(256)
+gated_rms_small_kernel(const float* __restrict__ x, const T* __restrict__ g, long long ldg,
+                       const float* __restrict__ w, T* __restrict__ out, int W, int groups, int gs,
+                       int SG, long long items, int shared_w, int gate_first, int sigmoid,
+                       float eps) {
+  const long long item = (blockIdx.x * 256ll + threadIdx.x) / SG;
+  const int c = 4 * (threadIdx.x & (SG - 1));
+  const bool on = item < items && c < gs;
+  const long long r = on ? item / groups : 0;
+  const int col = on ? (int)(item - r * groups) * gs + c : 0;
+  float v[4] = {0.f, 0.f, 0.f, 0.f}, z[4] = {0.f, 0.f, 0.f, 0.f};
+  if (on) {
+    load4<float>(x + r * W + col, v);
+    load4<T>(g + r * ldg + col, z);
+  }
+#pragma unroll
+  for (int e = 0; e < 4; ++e) z[e] = sigmoid ? sigmoid_f(z[e]) : silu_f(z[e]);
+  if (gate_first) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] *= z[e];
+  }
+  float ss = (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+  for (int m = 1; m < SG; m <<= 1) ss += __shfl_xor(ss, m, 64);
+  if (!on) return;
+  const float inv = 1.f / sqrtf(ss / (float)gs + eps);
+  float ww[4];
+  load4<float>(w + (shared_w ? c : col), ww);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) v[e] = v[e] * inv * ww[e] * (gate_first ? 1.f : z[e]);
+  store4<T>(out + r * W + col, v);
 }
 
 template <typename T>
@@ -217,20 +249,31 @@ hipError_t sm_group_rms(int dt_in, int dt_out, const void* x, long long ldx, con
 }
 
 // x fp32 [rows][W] contiguous; g [rows][W] with row stride ldg; w fp32 [W], or [W / groups] with
-// shared_w; out [rows][W] contiguous.  W * 4 bytes of LDS.
+// shared_w; out [rows][W] contiguous.
 hipError_t sm_gated_rms(int dt, const float* x, const void* g, long long ldg, const float* w,
                         void* out, int rows, int W, int groups, int shared_w, int gate_first,
                         int sigmoid, float eps, hipStream_t st) {
   if (rows == 0) return hipSuccess;
-  if (groups < 1 || W < 1 || W % groups || (size_t)W * sizeof(float) > 65536 - 64)
-    return hipErrorInvalidValue;
+  if (groups < 1 || W < 1 || W % groups) return hipErrorInvalidValue;
+  const int per = groups < 4 ? groups : 4;     // groups of one workgroup
+  const size_t lds = (size_t)(W / groups) * per * sizeof(float);
+  if (lds > 65536 - 64) return hipErrorInvalidValue;
+  const dim3 grid(rows, (groups + per - 1) / per);
   const bool vec = (W / groups) % 4 == 0 && ldg % 4 == 0 && (uintptr_t)x % 16 == 0 &&
                    (uintptr_t)g % 16 == 0 && (uintptr_t)out % 16 == 0;
-  const size_t lds = (size_t)W * sizeof(float);
+  const int gs = W / groups;
+  const bool small = vec && gs <= 256 && (uintptr_t)w % 16 == 0 && W % 4 == 0;
+  int SG = 1;
+  while (4 * SG < gs) SG <<= 1;
+  const long long items = (long long)rows * groups;
+  const unsigned blocks = (unsigned)((items * SG + 255) / 256);
 #define CALL(TT)                                                                                \
-  if (vec) gated_rms_kernel<TT, true><<<rows, 256, lds, st>>>(x, (const TT*)g, ldg, w, (TT*)out, \
+  if (small)                                                                                    \
+    gated_rms_small_kernel<TT><<<blocks, 256, 0, st>>>(x, (const TT*)g, ldg, w, (TT*)out, W,    \
+                                groups, gs, SG, items, shared_w, gate_first, sigmoid, eps);     \
+  else if (vec) gated_rms_kernel<TT, true><<<grid, 256, lds, st>>>(x, (const TT*)g, ldg, w, (TT*)out, \
                                                 W, groups, shared_w, gate_first, sigmoid, eps); \
-  else gated_rms_kernel<TT, false><<<rows, 256, lds, st>>>(x, (const TT*)g, ldg, w, (TT*)out, W, \
+  else gated_rms_kernel<TT, false><<<grid, 256, lds, st>>>(x, (const TT*)g, ldg, w, (TT*)out, W, \
                                                 groups, shared_w, gate_first, sigmoid, eps)
   SM_DISPATCH(dt, CALL)
 #undef CALL
