@@ -28,6 +28,9 @@
 //
 // Every spin has a deadline (s_memrealtime, 100 MHz). A rank whose peer never arrives sets
 // `err` and leaves, so a missing peer turns into a host-visible error instead of a hung GPU.
+// Once `err` is set, later barriers of that rank wait 1 ms at most: the ranks' epochs are out of
+// step then (a slot holds a later epoch than the one waited for and never returns to it), so
+// every further barrier of the launches still queued would run into the deadline as well.
 // The same timeout also sets a word in pinned, host-mapped memory (`host_err`), so the host
 // can poll it after every step with a plain load -- no device sync, no copy -- and stop before
 // it hands out tokens computed from a half-reduced tensor.
@@ -84,7 +87,9 @@ __device__ __forceinline__ void block_barrier(const Peers& P, Signal* self, int 
     uint64_t waited = 0;
     while (__hip_atomic_load(mine, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_SYSTEM) != epoch) {
       waited = __builtin_amdgcn_s_memrealtime() - t0;
-      if (waited > deadline_ticks) {
+      if (waited > deadline_ticks ||
+          (waited > kLongWaitTicks && __hip_atomic_load(&self->err, __ATOMIC_RELAXED,
+                                                        __HIP_MEMORY_SCOPE_SYSTEM) != 0u)) {
         __hip_atomic_fetch_or(&self->err, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_SYSTEM);
         uint32_t expect = 0u;
         const uint32_t info = (1u << 31) | ((uint32_t)slot << 24) | ((uint32_t)b << 16) |

@@ -325,9 +325,10 @@ class CustomAllReduce:
         torch.cuda.synchronize(self.device)
         for p in self._opened:
             self.C.car_close(p)
-        for p in (self._buf, self._sig):
-            if p is not None:
-                self.C.car_free(p)
+        # uncached allocations stay until the process ends (freeing one that a kernel has read can
+        # leave later tensors with wrong values on this platform); the signal block is always one
+        if self._buf is not None and self.cached:
+            self.C.car_free(self._buf)
         self._buf = self._sig = None
         self._opened = []
         self.data, self.sig = [], []
