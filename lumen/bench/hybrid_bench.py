@@ -4,10 +4,10 @@ Silonex) beside Llama at equal size.
 ``python bench.py --hybrid [--hybrid_family dalavik|fanopel|foderax|silonex]`` (one GPU).  Fanopel also
 runs beside the closest design the framework already had: a Gedatar stack of attention layers
 (keys as values) with routed experts of the same shapes; Foderax beside Dalavik (latent and
-grouped-query attention through the same row kernels) and Fanopel (experts of the same shapes); Silonex
-beside Gedatar (matrix-state recurrences of the same head sizes, dense feed-forwards) and Fanopel
-(window attention through the same kernels).  All models get random
-weights of layer shapes that resemble real models (width 2048 / 4096, head size 128 / 64, FFN 2.75 x width, vocab 32000), the
+grouped-query attention through the same row kernels) and Fanopel (experts of the same shapes);
+Silonex beside Gedatar (matrix-state recurrences of the same head sizes, dense feed-forwards) and
+Fanopel (window attention through the same kernels).  All models get random weights of layer shapes
+that resemble real models (width 2048 / 4096, head size 128 / 64, FFN 2.75 x width, vocab 32000), the
 same depth, and run the same forced-token workload through the serving engine
 (``lumen.serve.trace.TraceReplay``: the engine's input builder, block manager, state slots,
 runner, hipGraph decode):

@@ -75,13 +75,14 @@ CONFIGS = {
         _par((3, 3, 10, 14, 6), (3, 1, 9, 11, 1), None, 21, cap=None, scaling=None),
         _lin(3, 11, 7, [0.3, 1.0, 0.97], 33),
         _ssd(2, 5, 37, 2, 1, 5, None)]),
-    # one of everything: one copy, one head, one group, no loop, a window of one token, a factor of 1
+    # one of everything: one copy, one head, one group, no loop, a window of one token, a logit
+    # factor of 1
     "one": lambda: _cfg("one", 64, 48, 1, None, 1.0, 1e-4, [
         _lin(1, 16, 16, [0.9], 40),
         _par((1, 1, 16, 16, 16), (1, 1, 16, 16, 2), 24, 1),
         _ssd(1, 16, 16, 1, 1, 2, 24)]),
-    # head sizes 64 and 128 (the matrix-core attention's shapes), wide states, four copies, the whole
-    # stack looped, a window across tiles
+    # head sizes 64 and 128 (the matrix-core attention's shapes), wide states, four copies, the
+    # whole stack looped, a window across tiles
     "wide": lambda: _cfg("wide", 200, 128, 4, {"start": 0, "stop": 3, "times": 2}, 2.5, 1e-5, [
         _par((4, 1, 64, 64, 64), (2, 1, 128, 128, 4), 160, 70, base=500000.0, scale=0.12),
         _ssd(4, 64, 128, 1, 4, 4, 96),
@@ -115,8 +116,8 @@ oracle = Oracle
 def yardstick(orc, toks, want):
     """[T] how far rounding alone moves each position's logits: the oracle's own arithmetic in fp32
     against float64, and float64 with the embeddings moved by 3e-7 of themselves.  A norm over a
-    read-out that happens to be nearly zero magnifies rounding at that position a thousandfold, in any
-    implementation."""
+    read-out that happens to be nearly zero magnifies rounding at that position a thousandfold, in
+    any implementation."""
     g = torch.Generator().manual_seed(99)
     e = orc.w["embed"].to(ref.F64)
     moved = dict(orc.w, embed=e * (1.0 + 3e-7 * torch.randn(e.shape, generator=g, dtype=ref.F64)))
@@ -129,8 +130,10 @@ def check_conditioned(got, want, stick, rtol=2e-4):
     per = (got.to(ref.F64) - want).abs().max(-1).values
     limit = torch.clamp(8.0 * stick, min=rtol * max(float(want.std()), 1.0))
     t = int((per / limit).argmax())
-    assert float(per[t]) <= float(limit[t]), f"position {t}: {float(per[t]):.3e} > {float(limit[t]):.3e}"
-    assert float((stick > 4 * rtol).double().mean()) <= 0.1, "the weights make most rows ill-conditioned"
+    e, most = float(per[t]), float(limit[t])
+    assert e <= most, f"position {t}: {e:.3e} > {most:.3e}"
+    share = float((stick > 4 * rtol).double().mean())
+    assert share <= 0.1, f"the weights make {share:.0%} of the rows ill-conditioned"
 
 
 def close_to_rounding(m, toks, want, *gots):
@@ -268,8 +271,8 @@ def test_every_constant_counts(device, name):
 
     right, ssd = f"l{ip}.mix.right.", f"l{im}.mix."
     changes = {
-        "window + 1": cfg_with(lambda c: set_(left(c)["mask"], "size", left(c)["mask"]["size"] + 1)),
-        "window - 1": cfg_with(lambda c: set_(left(c)["mask"], "size", left(c)["mask"]["size"] - 1)),
+        "window + 1": cfg_with(lambda c: left(c)["mask"].update(size=left(c)["mask"]["size"] + 1)),
+        "window - 1": cfg_with(lambda c: left(c)["mask"].update(size=left(c)["mask"]["size"] - 1)),
         "soft cap": cfg_with(lambda c: set_(left(c), "softcap", None)),
         "stretch": cfg_with(lambda c: set_(left(c)["rot"], "scaling", None)),
         "scale": cfg_with(lambda c: set_(left(c), "scale", left(c)["scale"] * 0.9)),
@@ -277,7 +280,8 @@ def test_every_constant_counts(device, name):
         "norm groups": cfg_with(lambda c: set_(
             c["layers"][im]["mixer"], "norm_groups", 1)),
         "lightning decay": cfg_with(lambda c: set_(
-            c["layers"][il]["mixer"], "decay", [d * 0.95 for d in c["layers"][il]["mixer"]["decay"]])),
+            c["layers"][il]["mixer"], "decay",
+            [d * 0.95 for d in c["layers"][il]["mixer"]["decay"]])),
         "logit scale": cfg_with(lambda c: set_(c, "logit_scale", 1.0)),
         "skip": w_with(ssd + "D", lambda t: t * 0.0),
         "ssd decay": w_with(ssd + "A_log", lambda t: t + 0.3),
@@ -474,11 +478,13 @@ def _random_config(seed):
             layers.append(_lin(H, D, Dv, [rng.choice([0.4, 0.9, 0.99, 1.0]) for _ in range(H)], ff))
         else:
             n = rng.choice([x for x in (1, 2, 3, 4) if (H * Dv) % x == 0])
-            layers.append(_ssd(H, Dv, rng.choice([8, 16, 36, 64]), G, n, rng.choice([2, 3, 4, 6]), ff))
+            layers.append(_ssd(H, Dv, rng.choice([8, 16, 36, 64]), G, n, rng.choice([2, 3, 4, 6]),
+                               ff))
     a = rng.randint(0, len(layers) - 1)
     loop = {"start": a, "stop": rng.randint(a, len(layers)), "times": rng.randint(1, 3)}
     return _cfg(f"random{seed}", rng.randint(50, 400), W, rng.choice([1, 2, 3, 4]),
-                rng.choice([None, loop]), rng.choice([0.5, 1.0, 3.0]), rng.choice([1e-6, 1e-5]), layers)
+                rng.choice([None, loop]), rng.choice([0.5, 1.0, 3.0]), rng.choice([1e-6, 1e-5]),
+                layers)
 
 
 @pytest.mark.parametrize("device", DEVICES)
