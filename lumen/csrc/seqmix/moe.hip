@@ -12,7 +12,10 @@
 //                  get s / (sum of the chosen s + eps) * scale.  One wave per row, the row's c in
 //                  LDS; every arg-max breaks ties towards the lowest index.
 //   sm_gated_act   act(gate) * up over stacked [gate | up] blocks (act: SiLU, ReLU, tanh-GELU or
-//                  squared ReLU), expert e's block scaled by the row's routing weight; fp32 math.
+//                  squared ReLU; or clamped: g sigmoid(slope g) (u + shift) with g = min(gate, limit),
+//                  u = clamp(up, -limit, limit)), expert e's block scaled by the row's routing weight
+//                  -- the activation's result, or with weigh_in the gate and up values that enter it
+//                  (an expert whose INPUT is weighted); fp32 math.
 //   sm_scaled_act  act(up) over stacked up blocks of experts without a gate, scaled the same way.
 //   sm_write_k     rows of the key projection into the paged key cache by slot.
 #include "seqmix.h"
@@ -30,6 +33,28 @@ __device__ __forceinline__ float gate_act(float g, int act) {
     return r * r;
   }
   return act == 0 ? silu_f(g) : act == 1 ? fmaxf(g, 0.f) : gelu_tanh_f(g);
+}
+
+struct GateForm {
+  int act;                                  // as above; 4: clamped, with the constants below
+  int weigh_in;                             // the weight multiplies gate and up, not the result
+  float limit, limit_s, slope, shift;       // limit: experts; limit_s: the unweighted block
+};
+
+// the gated activation of one (gate, up) pair with routing weight w
+__device__ __forceinline__ float gated_f(float g, float u, float w, bool shared,
+                                         const GateForm& f) {
+  if (f.weigh_in) { g *= w; u *= w; }
+  float y;
+  if (f.act == 4) {
+    const float lim = shared ? f.limit_s : f.limit;
+    g = fminf(g, lim);
+    u = fminf(fmaxf(u, -lim), lim);
+    y = g * sigmoid_f(f.slope * g) * (u + f.shift);
+  } else {
+    y = gate_act(g, f.act) * u;
+  }
+  return f.weigh_in ? y : y * w;
 }
 
 // wave-wide arg-max of (value, index) pairs, ties to the lowest index; every lane gets the result
@@ -220,7 +245,7 @@ route_topk_kernel(const float* __restrict__ z, float* __restrict__ out, int T, i
 template <typename T>
 __global__ void gated_act_kernel(const T* __restrict__ gu, const float* __restrict__ wts,
                                  T* __restrict__ out, int Tn, int E, int ff, int ffs,
-                                 int act) {
+                                 const GateForm form) {
   const int in_w = E * 2 * ff + 2 * ffs, out_w = E * ff + ffs;
   const long long n = (long long)Tn * out_w;
   for (long long i = blockIdx.x * (long long)blockDim.x + threadIdx.x; i < n;
@@ -238,7 +263,7 @@ __global__ void gated_act_kernel(const T* __restrict__ gu, const float* __restri
       g = to_f32(row[E * 2 * ff + q]);
       u = to_f32(row[E * 2 * ff + ffs + q]);
     }
-    out[i] = from_f32<T>(w == 0.f ? 0.f : gate_act(g, act) * u * w);
+    out[i] = from_f32<T>(w == 0.f ? 0.f : gated_f(g, u, w, c >= E * ff, form));
   }
 }
 
@@ -246,7 +271,7 @@ __global__ void gated_act_kernel(const T* __restrict__ gu, const float* __restri
 template <typename T>
 __global__ void __launch_bounds__(256)
 gated_act_v8(const T* __restrict__ gu, const float* __restrict__ wts, T* __restrict__ out, int Tn,
-             int E, int ff, int ffs, int act) {
+             int E, int ff, int ffs, const GateForm form) {
   const int in_w = E * 2 * ff + 2 * ffs, out_w = E * ff + ffs;
   const int c = 8 * (blockIdx.x * 256 + threadIdx.x);
   if (c >= out_w) return;
@@ -270,7 +295,7 @@ gated_act_v8(const T* __restrict__ gu, const float* __restrict__ wts, T* __restr
       load8<T>(row + goff, g);
       load8<T>(row + uoff, u);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) o[j] = gate_act(g[j], act) * u[j] * w;
+      for (int j = 0; j < 8; ++j) o[j] = gated_f(g[j], u[j], w, e < 0, form);
     }
     store8<T>(out + (long long)t * out_w + c, o);
   }
@@ -338,21 +363,24 @@ hipError_t sm_scaled_act(int dt, const void* u, const float* wts, void* out, int
 }
 
 hipError_t sm_gated_act(int dt, const void* gu, const float* wts, void* out, int T, int E, int ff,
-                        int ffs, int act, hipStream_t st) {
+                        int ffs, int act, int weigh_in, float limit, float limit_s, float slope,
+                        float shift, hipStream_t st) {
   const long long n = (long long)T * (E * ff + ffs);
   if (n == 0) return hipSuccess;
+  if (act < 0 || act > 4) return hipErrorInvalidValue;
+  const GateForm form{act, weigh_in, limit, limit_s, slope, shift};
   if (E > 0 && wts == nullptr) return hipErrorInvalidValue;
   if (ff % 8 == 0 && ffs % 8 == 0 && (dt == kBF16 || dt == kF16)) {
     const dim3 grid(((E * ff + ffs) / 8 + 255) / 256, T < 65535 ? T : 65535);
     if (dt == kBF16)
       gated_act_v8<bf16><<<grid, 256, 0, st>>>((const bf16*)gu, wts, (bf16*)out, T, E, ff, ffs,
-                                                 act);
+                                                 form);
     else
       gated_act_v8<fp16><<<grid, 256, 0, st>>>((const fp16*)gu, wts, (fp16*)out, T, E, ff, ffs,
-                                                 act);
+                                                 form);
     return hipGetLastError();
   }
-#define CALL(TT) gated_act_kernel<TT><<<grid_for(n), 256, 0, st>>>((const TT*)gu, wts, (TT*)out, T, E, ff, ffs, act)
+#define CALL(TT) gated_act_kernel<TT><<<grid_for(n), 256, 0, st>>>((const TT*)gu, wts, (TT*)out, T, E, ff, ffs, form)
   SM_DISPATCH(dt, CALL)
 #undef CALL
   return hipGetLastError();

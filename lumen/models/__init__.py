@@ -1,8 +1,10 @@
 """Model families: Llama / Llama-2 (7B, 13B, 70B-GQA), OPT (125m), Gedatar (hybrid stack),
 Dalavik (latent + grouped-query attention stack), Fanopel (gated window attention + routed
 experts), Foderax (parallel sigmoid-attention / minGRU, latent and differential attention
-layers with routed experts and depth-weighted layer inputs) and Silonex (window attention beside
-a gated delta rule, lightning attention, state-space duality; hyper-connections, looped layers)."""
+layers with routed experts and depth-weighted layer inputs), Silonex (window attention beside
+a gated delta rule, lightning attention, state-space duality; hyper-connections, looped layers) and
+Tazulix (whole-projection normed attention beside lightning attention, experts that weigh their
+input; looped layers that read the embedding anew)."""
 from __future__ import annotations
 
 from typing import Optional
@@ -17,11 +19,13 @@ from .gedatar import GedatarForCausalLM  # noqa: F401
 from .llama import LlamaForCausalLM  # noqa: F401
 from .opt import OPTForCausalLM  # noqa: F401
 from .silonex import SilonexForCausalLM  # noqa: F401
+from .tazulix import TazulixForCausalLM  # noqa: F401
 
 
 MODEL_CLASSES = {"llama": LlamaForCausalLM, "opt": OPTForCausalLM, "gedatar": GedatarForCausalLM,
                  "dalavik": DalavikForCausalLM, "fanopel": FanopelForCausalLM,
-                 "foderax": FoderaxForCausalLM, "silonex": SilonexForCausalLM}
+                 "foderax": FoderaxForCausalLM, "silonex": SilonexForCausalLM,
+                 "tazulix": TazulixForCausalLM}
 
 
 def build_model(name_or_cfg, dtype=torch.bfloat16, device=None, init: str = "auto",

@@ -17,7 +17,8 @@ from typing import Optional
 
 @dataclass
 class ModelConfig:
-    arch: str = "llama"  # "llama" | "opt" | "gedatar" | "dalavik" | "fanopel" | "foderax" | "silonex"
+    # "llama" | "opt" | "gedatar" | "dalavik" | "fanopel" | "foderax" | "silonex" | "tazulix"
+    arch: str = "llama"
     vocab_size: int = 32000
     hidden_size: int = 4096
     intermediate_size: int = 11008
@@ -57,7 +58,8 @@ class ModelConfig:
     logit_softcap: float = 0.0
     # Silonex (layer_specs of "parallel" | "lightning" | "mamba2" mixers): copies of the residual
     # stream, the layers that run several times in a row ({"start", "stop", "times"} or None) and
-    # the factor of the logits
+    # the factor of the logits.  Tazulix (layer_specs of "attention" | "lightning" mixers, dense or
+    # routed feed-forwards) has ``loop`` and ``embedding_scale``
     streams: int = 1
     loop: Optional[dict] = None
     logit_scale: float = 1.0
@@ -66,7 +68,8 @@ class ModelConfig:
     def is_hybrid(self) -> bool:
         """Every layer names its own mixer and keeps its own kind of cache or state; such a stack
         is served by ``serve.hybrid_runner`` on the step's row segments."""
-        return self.arch in ("gedatar", "dalavik", "fanopel", "foderax", "silonex")
+        return self.arch in ("gedatar", "dalavik", "fanopel", "foderax", "silonex",
+                             "tazulix")
 
     @property
     def head_dim(self) -> int:
@@ -92,6 +95,8 @@ class ModelConfig:
                 from .foderax import tensor_shapes
             elif self.arch == "silonex":
                 from .silonex import tensor_shapes
+            elif self.arch == "tazulix":
+                from .tazulix import tensor_shapes
             else:
                 from .dalavik import tensor_shapes
 
@@ -283,7 +288,41 @@ def silonex_to_dict(cfg: ModelConfig) -> dict:
     return d
 
 
+def _tazulix_to_config(d: dict) -> ModelConfig:
+    """config.json of a Tazulix checkpoint: {"architecture": "Tazulix", "vocab", "width",
+    "embedding": {"scale"}, "loop": {"start", "stop", "times"}, "norm": {"eps"}, "layers":
+    [{"type", "mixer", "mlp"}, ...]}."""
+    layers = d["layers"]
+    if not layers:
+        raise ValueError("a Tazulix config needs at least one layer")
+    for i, L in enumerate(layers):
+        if L.get("type") not in ("attention", "lightning"):
+            raise ValueError(f"layer {i}: unknown mixer type {L.get('type')!r}")
+        if L.get("mlp") and L["mlp"].get("kind") not in ("dense", "moe"):
+            raise ValueError(f"layer {i}: unknown feed-forward kind {L['mlp'].get('kind')!r}")
+    return ModelConfig(
+        arch="tazulix", vocab_size=int(d["vocab"]), hidden_size=int(d["width"]),
+        num_hidden_layers=len(layers), rms_norm_eps=float(d["norm"]["eps"]),
+        embedding_scale=float((d.get("embedding") or {}).get("scale", 1.0)),
+        loop=d.get("loop") or None, layer_specs=layers, intermediate_size=0,
+        num_attention_heads=0, num_key_value_heads=0, max_position_embeddings=1 << 20,
+        bos_token_id=int(d.get("bos_token_id", 0)), eos_token_id=int(d.get("eos_token_id", -1)),
+        pad_token_id=int(d.get("pad_token_id", 0)), name=d.get("_name_or_path", "tazulix"))
+
+
+def tazulix_to_dict(cfg: ModelConfig) -> dict:
+    """The checkpoint form of a Tazulix configuration (inverse of ``_tazulix_to_config``)."""
+    d = {"architecture": "Tazulix", "vocab": cfg.vocab_size, "width": cfg.hidden_size,
+         "embedding": {"scale": cfg.embedding_scale}, "norm": {"eps": cfg.rms_norm_eps},
+         "layers": cfg.layer_specs, "eos_token_id": cfg.eos_token_id}
+    if cfg.loop:
+        d["loop"] = cfg.loop
+    return d
+
+
 def _hf_to_config(d: dict) -> ModelConfig:
+    if d.get("architecture") == "Tazulix":
+        return _tazulix_to_config(d)
     if d.get("architecture") == "Silonex":
         return _silonex_to_config(d)
     if d.get("architecture") == "Foderax":
@@ -484,6 +523,31 @@ PRESETS = {
             {"type": "mamba2", "mixer": {"heads": 4, "vdim": 32, "state": 16, "groups": 1,
                                          "norm_groups": 1, "conv": 2},
              "mlp": {"kind": "dense", "ff": 96}}]),
+    # whole-projection q / k norms, YaRN rotary and biases beside lightning attention; dense and
+    # routed (input-weighted, clamped experts) feed-forwards, one layer without; a looped pair of
+    # layers that reads the embedding anew at every pass
+    "tiny-tazulix": dict(
+        arch="tazulix", vocab_size=344, hidden_size=104, num_hidden_layers=4, rms_norm_eps=1e-5,
+        embedding_scale=7.5, loop={"start": 1, "stop": 3, "times": 3}, intermediate_size=0,
+        num_attention_heads=0, num_key_value_heads=0, max_position_embeddings=1 << 20,
+        eos_token_id=-1, name="tiny-tazulix", layer_specs=[
+            {"type": "lightning", "mixer": {"heads": 3, "dim": 24, "vdim": 16,
+                                            "decay": [0.5, 0.9, 0.99]},
+             "mlp": {"kind": "dense", "ff": 168}},
+            {"type": "attention", "mixer": {
+                "heads": 6, "kv_heads": 2, "dim": 32, "vdim": 24, "scale": 0.2,
+                "rot": {"base": 5000.0, "dims": 24,
+                        "scaling": {"factor": 8.0, "original": 128, "fast": 16.0, "slow": 1.0}}},
+             "mlp": {"kind": "moe", "router": {"experts": 6, "top": 2},
+                     "expert": {"ff": 40, "limit": 0.8}, "shared": {"ff": 72, "limit": 1.5}}},
+            {"type": "lightning", "mixer": {"heads": 2, "dim": 16, "vdim": 40,
+                                            "decay": [0.8, 0.999]},
+             "mlp": None},
+            {"type": "attention", "mixer": {
+                "heads": 3, "kv_heads": 3, "dim": 16, "vdim": 32, "scale": 0.3,
+                "rot": {"base": 20000.0, "dims": 16}},
+             "mlp": {"kind": "moe", "router": {"experts": 5, "top": 1},
+                     "expert": {"ff": 56, "limit": 2.0}, "shared": {"ff": 32, "limit": 0.5}}}]),
     "tiny-opt": dict(arch="opt", vocab_size=512, hidden_size=64, intermediate_size=256,
                      ffn_dim=256, num_hidden_layers=2, num_attention_heads=4,
                      num_key_value_heads=4, max_position_embeddings=256, word_embed_proj_dim=64,

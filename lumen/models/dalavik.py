@@ -169,22 +169,3 @@ class DalavikForCausalLM(NamedTensorModel):
         if input_ids.dim() == 1:
             input_ids = input_ids.view(1, -1)
         return forward_fresh(self, input_ids)
-
-
-@torch.no_grad()
-def load_dalavik_weights(model: DalavikForCausalLM, handles: dict, path: str) -> None:
-    """Every tensor the configuration implies must be in the checkpoint with its shape; tensors
-    the configuration has no use for are listed in ``model.ignored_tensors`` and not read."""
-    names = model.tensor_names()
-    missing = sorted(set(names) - set(handles))
-    if missing:
-        raise KeyError(f"{path}: missing tensors {missing[:8]}")
-    model.ignored_tensors = sorted(set(handles) - set(names))
-    for name in names:
-        t = handles[name].get_tensor(name)
-        dst = model.tensor(name)
-        if tuple(t.shape) != tuple(dst.shape):
-            raise ValueError(f"{name}: checkpoint {tuple(t.shape)} != model {tuple(dst.shape)}")
-        if not t.is_floating_point():
-            raise ValueError(f"{name}: expected a floating-point tensor, got {t.dtype}")
-        dst.copy_(t.to(dst.dtype))

@@ -75,22 +75,10 @@ def load_hf_weights(model: nn.Module, path: str, strict: bool = True) -> None:
         from .gedatar import load_gedatar_weights
 
         return load_gedatar_weights(model, handles, path)
-    if model.config.arch == "dalavik":
-        from .dalavik import load_dalavik_weights
+    if model.config.is_hybrid:
+        from .named import load_named_weights
 
-        return load_dalavik_weights(model, handles, path)
-    if model.config.arch == "fanopel":
-        from .fanopel import load_fanopel_weights
-
-        return load_fanopel_weights(model, handles, path)
-    if model.config.arch == "foderax":
-        from .foderax import load_foderax_weights
-
-        return load_foderax_weights(model, handles, path)
-    if model.config.arch == "silonex":
-        from .silonex import load_silonex_weights
-
-        return load_silonex_weights(model, handles, path)
+        return load_named_weights(model, handles, path)
     params = dict(model.named_parameters())
     for ours, srcs in _hf_name_map(model).items():
         if ours not in params:
@@ -121,14 +109,14 @@ def save_hf_weights(model: nn.Module, path: str, shard_bytes: int = 5 << 30) -> 
     cfg = model.config
     if cfg.is_hybrid:
         from .config import (dalavik_to_dict, fanopel_to_dict, foderax_to_dict, gedatar_to_dict,
-                             silonex_to_dict)
+                             silonex_to_dict, tazulix_to_dict)
 
         save_file({n: model.tensor(n).detach().cpu().contiguous() for n in model.tensor_names()},
                   os.path.join(path, "model.safetensors"), metadata={"format": "pt"})
         with open(os.path.join(path, "config.json"), "w") as f:
             to_dict = {"gedatar": gedatar_to_dict, "dalavik": dalavik_to_dict,
                        "fanopel": fanopel_to_dict, "foderax": foderax_to_dict,
-                       "silonex": silonex_to_dict}[cfg.arch]
+                       "silonex": silonex_to_dict, "tazulix": tazulix_to_dict}[cfg.arch]
             json.dump(to_dict(cfg), f, indent=2)
         return
     params = dict(model.named_parameters())

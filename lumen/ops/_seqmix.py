@@ -32,7 +32,7 @@ SIGNATURES = {
     "sm_chunk_attn": "iplpppippiiiiiffii",
     "sm_chunk_attn_tiles": "iplpppipippiiiiffiii",
     "sm_route_topk": "ppiii",
-    "sm_gated_act": "ipppiiiii",
+    "sm_gated_act": "ipppiiiii" "iffff",
     "sm_group_rms": "iiplpppliiif",
     "sm_gate_rows": "iplplpiipi",
     "sm_rotate_heads": "iplliiippi",
@@ -56,6 +56,8 @@ SIGNATURES = {
     "sm_gated_rms": "ipplppiiiiiif",
     "sm_hyper_mix": "i" "pppi" "ppppf" "ppp" "ppf" "pp" "iiii",
     "sm_head_norm_rotary": "ipl" "ppppppp" "iiiiiiif",
+    "sm_row_norm_rotary": "ipl" "ppppppp" "iiiiii" "ff",
+    "sm_stream_rms": "ipi" "ppif" "p" "pppf" "ppi" "iif",
     "sm_head_scan_chunk": "ii" "plplplplpl" "pppp" "pp" "ppp" "iiiiiiff",
     "sm_head_scan_step": "ii" "plplplplpl" "pppp" "pp" "ppp" "iiiiiiff",
     "sm_short_conv": "iplpppp" "pppp" "iii",

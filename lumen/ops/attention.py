@@ -769,6 +769,64 @@ def row_norm_write(qk: torch.Tensor, wq: torch.Tensor, wk: torch.Tensor, slots: 
          qk.shape[0], HD, GD, eps)
 
 
+def row_norm_rotary_write_ref(z, wq, wk, positions, slots, kcache, vcache, H, G, D, Dv, dims,
+                              inv_freq, amp, eps):
+    T = z.shape[0]
+
+    def unit(x):
+        return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
+
+    def turn(x):
+        if not dims:
+            return x
+        a = positions.float().view(T, 1, 1) * inv_freq.float().view(1, 1, -1)
+        c, s = torch.cos(a) * amp, torch.sin(a) * amp
+        u, v = x[..., :dims // 2], x[..., dims // 2:dims]
+        return torch.cat([u * c - v * s, v * c + u * s, x[..., dims:]], -1)
+
+    q = turn((unit(z[:, :H * D].float()) * wq.float()).view(T, H, D))
+    k = turn((unit(z[:, H * D:(H + G) * D].float()) * wk.float()).view(T, G, D))
+    v = z[:, (H + G) * D:(H + G) * D + G * Dv]
+    z[:, :H * D] = q.reshape(T, H * D).to(z.dtype)
+    ok = slots >= 0
+    kcache.view(-1, G, D)[slots[ok]] = k[ok].to(kcache.dtype)
+    vcache.view(-1, G * Dv)[slots[ok]] = v[ok].to(vcache.dtype)
+
+
+def row_norm_rotary_write(z: torch.Tensor, wq: torch.Tensor, wk: torch.Tensor,
+                          positions: torch.Tensor, slots: torch.Tensor, kcache: torch.Tensor,
+                          vcache: torch.Tensor, H: int, G: int, D: int, Dv: int, dims: int,
+                          inv_freq: torch.Tensor, amp: float, eps: float) -> None:
+    """z [T, >= (H + G) * D + G * Dv] (a fused projection's output [q | k | v]; further columns are
+    left alone): the query part is RMS-normed over ALL its H * D entries at once with the weight
+    ``wq`` [H * D], the key part over its G * D with ``wk`` [G * D]; then every head is turned on its
+    first ``dims`` entries in the half layout by position * ``inv_freq``, cosine and sine multiplied
+    by ``amp``.  q is replaced in place, k and the values as projected go to their paged caches
+    [blocks, block, G, D] / [.., G, Dv] at ``slots`` (int64; -1 skips).  Norms, angles and rotation
+    are fp32.  (HIP: ``csrc/seqmix/row_rotary.hip``.)"""
+    from ._seqmix import DT, call, use_seqmix
+
+    if dims % 2 or dims > D:
+        raise ValueError(f"rotary dims {dims} must be even and at most the head size {D}")
+    if z.shape[1] < (H + G) * D + G * Dv:
+        raise ValueError(f"z has {z.shape[1]} columns, expected at least {(H + G) * D + G * Dv}")
+    if tuple(kcache.shape[2:]) != (G, D) or tuple(vcache.shape[2:]) != (G, Dv):
+        raise ValueError(f"caches {tuple(kcache.shape)} / {tuple(vcache.shape)} do not hold {G} "
+                         f"heads of {D} / {Dv}")
+    if wq.numel() != H * D or wk.numel() != G * D:
+        raise ValueError(f"norm weights of {wq.numel()} / {wk.numel()} for parts of {H * D} / "
+                         f"{G * D}")
+    if not use_seqmix(z):
+        return row_norm_rotary_write_ref(z, wq, wk, positions, slots, kcache, vcache, H, G, D, Dv,
+                                         dims, inv_freq, amp, eps)
+    assert z.stride(1) == 1 and kcache.is_contiguous() and vcache.is_contiguous()
+    assert kcache.dtype == z.dtype and vcache.dtype == z.dtype and positions.dtype == torch.int32
+    assert wq.dtype == torch.float32 and wk.dtype == torch.float32
+    assert inv_freq.dtype == torch.float32 and inv_freq.numel() >= dims // 2
+    call("sm_row_norm_rotary", DT[z.dtype], z, z.stride(0), wq, wk, positions, slots, kcache,
+         vcache, inv_freq, z.shape[0], H, G, D, G * Dv, dims, float(amp), eps)
+
+
 def row_attention_ref(q1, q2, kcache, vcache, Dv, out, seg, H, G, scale, softcap=0.0,
                       q_temp=None, r1=None, r2=None, talk=None, sink=None, slopes=None,
                       window=0, keep_first=0, gate=None, sigmoid_bias=None, v_div=1):

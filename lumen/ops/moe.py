@@ -20,7 +20,8 @@ projections side by side in one [W, E * ff + ffs] weight):
 """
 from __future__ import annotations
 
-from typing import Optional
+from dataclasses import dataclass
+from typing import Optional, Union
 
 import torch
 import torch.nn.functional as F
@@ -115,32 +116,60 @@ _ACT_FN = {"silu": F.silu, "relu": F.relu, "gelu_tanh": lambda z: F.gelu(z, appr
            "relu2": lambda z: F.relu(z) ** 2}
 
 
-def gated_act_ref(gu, wts, E, ff, ffs, act="silu"):
+@dataclass(frozen=True)
+class ClampedGate:
+    """The gated activation g * sigmoid(slope * g) * (u + shift) with g = min(gate, limit) and
+    u = clamp(up, -limit, limit); the unweighted block (the shared expert) has ``limit_shared``."""
+    limit: float
+    limit_shared: float
+    slope: float = 1.0
+    shift: float = 0.0
+
+
+def gated_act_ref(gu, wts, E, ff, ffs, act="silu", weigh="output"):
     T = gu.shape[0]
-    fn = _ACT_FN[act]
+
+    def pair(g, u, limit):
+        if isinstance(act, str):
+            return _ACT_FN[act](g) * u
+        g, u = torch.clamp(g, max=limit), torch.clamp(u, min=-limit, max=limit)
+        return g * torch.sigmoid(act.slope * g) * (u + act.shift)
+
+    lim, lim_s = (0.0, 0.0) if isinstance(act, str) else (act.limit, act.limit_shared)
     parts = []
     if E:
         g = gu[:, :E * 2 * ff].float().view(T, E, 2, ff)
-        parts.append((fn(g[:, :, 0]) * g[:, :, 1] * wts.float()[:, :, None]).reshape(T, E * ff))
+        wt = wts.float()[:, :, None]
+        y = (pair(g[:, :, 0] * wt, g[:, :, 1] * wt, lim) if weigh == "input"
+             else pair(g[:, :, 0], g[:, :, 1], lim) * wt)
+        parts.append(y.reshape(T, E * ff))
     if ffs:
         s = gu[:, E * 2 * ff:].float().view(T, 2, ffs)
-        parts.append(fn(s[:, 0]) * s[:, 1])
+        parts.append(pair(s[:, 0], s[:, 1], lim_s))
     return torch.cat(parts, 1).to(gu.dtype)
 
 
 def gated_act(gu: torch.Tensor, wts: Optional[torch.Tensor], E: int, ff: int,
-              ffs: int, act: str = "silu") -> torch.Tensor:
+              ffs: int, act: Union[str, ClampedGate] = "silu",
+              weigh: str = "output") -> torch.Tensor:
     """act(gate) * up over stacked [gate | up] blocks (``act``: silu, i.e. SwiGLU, relu or
-    gelu_tanh): ``gu`` [T, E * 2 * ff + 2 * ffs] holds E expert blocks (gate rows then up rows,
-    ff each) and one unweighted block of ffs (a dense feed-forward, or the shared expert);
-    expert e's activation is scaled by ``wts[:, e]``.  Returns [T, E * ff + ffs]."""
+    gelu_tanh, or a ``ClampedGate``): ``gu`` [T, E * 2 * ff + 2 * ffs] holds E expert blocks (gate
+    rows then up rows, ff each) and one unweighted block of ffs (a dense feed-forward, or the
+    shared expert); expert e's activation is scaled by ``wts[:, e]``, or with ``weigh`` = "input"
+    its gate and up values are (they are linear in the expert's input, so this is the expert of the
+    weighted input).  Returns [T, E * ff + ffs]."""
     from ._seqmix import DT, call, use_seqmix
 
+    if weigh not in ("output", "input"):
+        raise ValueError(f"unknown place of the routing weight {weigh!r}")
     if not use_seqmix(gu):
-        return gated_act_ref(gu, wts, E, ff, ffs, act)
+        return gated_act_ref(gu, wts, E, ff, ffs, act, weigh)
     assert gu.is_contiguous() and gu.shape[1] == E * 2 * ff + 2 * ffs
     out = torch.empty(gu.shape[0], E * ff + ffs, dtype=gu.dtype, device=gu.device)
-    call("sm_gated_act", DT[gu.dtype], gu, wts, out, gu.shape[0], E, ff, ffs, GATE_ACTS[act])
+    code, c = (GATE_ACTS[act], (0.0,) * 4) if isinstance(act, str) else (
+        4, (act.limit, act.limit_shared, act.slope, act.shift))
+    call("sm_gated_act", DT[gu.dtype], gu, wts, out, gu.shape[0], E, ff, ffs, code,
+         int(weigh == "input"), *c)
     return out
 
 
@@ -172,17 +201,21 @@ def scaled_act(u: torch.Tensor, wts: Optional[torch.Tensor], E: int, ff: int, ff
     return out
 
 
-def _act(z, wts, E, ff, ffs, act, gated):
-    return (gated_act if gated else scaled_act)(z, wts, E, ff, ffs, act)
+def _act(z, wts, E, ff, ffs, act, gated, weigh):
+    if gated:
+        return gated_act(z, wts, E, ff, ffs, act, weigh)
+    if weigh != "output":
+        raise ValueError("experts without a gate take their weight on the output")
+    return scaled_act(z, wts, E, ff, ffs, act)
 
 
-def moe_dense(h, wts, gu_w, down_w, E: int, ff: int, ffs: int, act: str = "silu",
-              gated: bool = True) -> torch.Tensor:
-    return F.linear(_act(F.linear(h, gu_w), wts, E, ff, ffs, act, gated), down_w)
+def moe_dense(h, wts, gu_w, down_w, E: int, ff: int, ffs: int, act="silu", gated: bool = True,
+              weigh: str = "output") -> torch.Tensor:
+    return F.linear(_act(F.linear(h, gu_w), wts, E, ff, ffs, act, gated, weigh), down_w)
 
 
-def moe_grouped(h, wts, gu_w, down_w, E: int, ff: int, ffs: int, act: str = "silu",
-                gated: bool = True) -> torch.Tensor:
+def moe_grouped(h, wts, gu_w, down_w, E: int, ff: int, ffs: int, act="silu", gated: bool = True,
+                weigh: str = "output") -> torch.Tensor:
     """Same result as ``moe_dense`` (to rounding) running each expert on its own rows only."""
     T = h.shape[0]
     k = 2 if gated else 1                                 # rows of the first weight per ff
@@ -198,13 +231,13 @@ def moe_grouped(h, wts, gu_w, down_w, E: int, ff: int, ffs: int, act: str = "sil
     for e, n in enumerate(counts):
         if n:
             gu = F.linear(x[a:a + n], gu_w[e * k * ff:(e + 1) * k * ff])
-            torch.matmul(_act(gu, None, 0, 0, ff, act, gated), down_w[:, e * ff:(e + 1) * ff].t(),
-                         out=ys[a:a + n])
+            torch.matmul(_act(gu, wsel[a:a + n], 1, ff, 0, act, gated, weigh),
+                         down_w[:, e * ff:(e + 1) * ff].t(), out=ys[a:a + n])
             a += n
-    out.index_add_(0, tok, ys.float() * wsel)
+    out.index_add_(0, tok, ys.float())
     if ffs:
         gu = F.linear(h, gu_w[E * k * ff:])
-        out += F.linear(_act(gu, None, 0, 0, ffs, act, gated), down_w[:, E * ff:]).float()
+        out += F.linear(_act(gu, None, 0, 0, ffs, act, gated, weigh), down_w[:, E * ff:]).float()
     return out.to(h.dtype)
 
 
@@ -215,8 +248,8 @@ def grouped_mm_ok(h: torch.Tensor, ff: int) -> bool:
             and hasattr(torch, "_grouped_mm") and ff % 8 == 0 and h.shape[1] % 8 == 0)
 
 
-def moe_grouped_mm(h, wts, gu_w, down_w, E: int, top: int, ff: int, ffs: int, act: str = "silu",
-                   gated: bool = True) -> torch.Tensor:
+def moe_grouped_mm(h, wts, gu_w, down_w, E: int, top: int, ff: int, ffs: int, act="silu",
+                   gated: bool = True, weigh: str = "output") -> torch.Tensor:
     """``moe_grouped`` without the host in the loop: every row has exactly ``top`` chosen
     experts, so the (row, expert) pairs are a [T * top] list of static size; sorted by expert they
     feed ONE grouped GEMM per projection whose group offsets stay on the device.  No
@@ -230,13 +263,14 @@ def moe_grouped_mm(h, wts, gu_w, down_w, E: int, top: int, ff: int, ffs: int, ac
     offs = torch.cumsum(torch.bincount(exp, minlength=E), 0).to(torch.int32)
     x = h.index_select(0, tok)
     u = torch._grouped_mm(x, gu_w[:E * k * ff].view(E, k * ff, W).transpose(1, 2), offs=offs)
-    a = _act(u, val.reshape(-1)[order].reshape(-1, 1).contiguous(), 1, ff, 0, act, gated)
+    a = _act(u, val.reshape(-1)[order].reshape(-1, 1).contiguous(), 1, ff, 0, act, gated,
+             weigh)
     y = torch._grouped_mm(a, down_w[:, :E * ff].view(W, E, ff).permute(1, 2, 0), offs=offs)
     out = torch.zeros(T, W, dtype=torch.float32, device=h.device)
     out.index_add_(0, tok, y.float())
     if ffs:
         gu = F.linear(h, gu_w[E * k * ff:])
-        out += F.linear(_act(gu, None, 0, 0, ffs, act, gated), down_w[:, E * ff:]).float()
+        out += F.linear(_act(gu, None, 0, 0, ffs, act, gated, weigh), down_w[:, E * ff:]).float()
     return out.to(h.dtype)
 
 
@@ -249,14 +283,17 @@ GROUPED_RATE_RATIO = 3
 GROUPED_MIN_SAVING = 32768          # rows x (E - GROUPED_RATE_RATIO * top)
 
 
-def moe(h, wts, gu_w, down_w, E: int, top: int, ff: int, ffs: int, act: str = "silu",
-        gated: bool = True) -> torch.Tensor:
+def moe(h, wts, gu_w, down_w, E: int, top: int, ff: int, ffs: int, act="silu",
+        gated: bool = True, weigh: str = "output") -> torch.Tensor:
     """Weighted sum of each row's chosen experts (+ the shared expert): [T, W] in h's dtype.
     ``gated``: an expert is W_down (act(W_gate h) * W_up h) with [gate | up] rows stacked per
-    expert in ``gu_w``; else W_down act(W_up h) with the up rows alone."""
+    expert in ``gu_w`` (``act`` also a ``ClampedGate``); else W_down act(W_up h) with the up rows
+    alone.  ``weigh`` = "input": an expert sees its weight times h instead of weighing in with its
+    output (gated experts)."""
     spare = E - GROUPED_RATE_RATIO * top
     grouped = (spare > 0 and h.shape[0] * spare >= GROUPED_MIN_SAVING
                and not (h.is_cuda and torch.cuda.is_current_stream_capturing()))
     if grouped and grouped_mm_ok(h, ff):
-        return moe_grouped_mm(h, wts, gu_w, down_w, E, top, ff, ffs, act, gated)
-    return (moe_grouped if grouped else moe_dense)(h, wts, gu_w, down_w, E, ff, ffs, act, gated)
+        return moe_grouped_mm(h, wts, gu_w, down_w, E, top, ff, ffs, act, gated, weigh)
+    return (moe_grouped if grouped else moe_dense)(h, wts, gu_w, down_w, E, ff, ffs, act, gated,
+                                                   weigh)

@@ -234,6 +234,84 @@ def weight_layer_norm(x: torch.Tensor, w: torch.Tensor, eps: float, out_dtype=No
     return scaled_residual_layer_norm(x, None, 0.0, w, eps, out_dtype or x.dtype, b)[1]
 
 
+# ---- pre-norm residual stream with RMS norms ---------------------------------------------------------
+# The fp32 stream takes what joins it and the same pass hands on the next sublayer's input,
+# h = x / sqrt(mean(x^2) + eps) * w in the compute dtype -- or, where a GEMM reads the stream itself,
+# its two 16-bit parts (rounded value, rounded remainder) as [2 T, W]: their products summed in fp32
+# keep about 16 bits of the stream's mantissa.  (HIP: ``csrc/seqmix/stream_rms.hip``.)
+SPLIT = "split"
+
+
+def rms_norm_rows_ref(x, w, eps, out_dtype):
+    return (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
+
+
+def _stream_rms(x, keep, out, eps, dtype, tokens=None, table=None, scale=1.0, y=None, f=(),
+                f2=None, coef=0.0):
+    """The new stream in ``x`` [T, W]; ``out``: a norm weight, SPLIT or None -> h, parts or None."""
+    from ._seqmix import DT, call, use_seqmix
+
+    split = isinstance(out, str)
+    w = None if split else out
+    if not use_seqmix(x):
+        v = x if keep else torch.zeros_like(x)
+        if table is not None:
+            v = v + table[tokens].float() * scale
+        for p in ([y] if y is not None else []) + list(f):
+            v = v + p.float()
+        if f2 is not None:
+            v = v + coef * f2
+        x.copy_(v)
+        if w is not None:
+            return rms_norm_rows_ref(x, w, eps, dtype)
+        if not split or dtype == torch.float32:
+            return x if split else None
+        hi = x.to(dtype)
+        return torch.cat([hi, (x - hi.float()).to(dtype)], 0)
+    T, W = x.shape
+    assert x.dtype == torch.float32 and x.is_contiguous() and len(f) <= 2
+    assert y is None or (y.is_contiguous() and y.dtype == dtype and tuple(y.shape) == (T, W))
+    for p in tuple(f) + ((f2,) if f2 is not None else ()):
+        assert p.dtype == torch.float32 and p.is_contiguous() and tuple(p.shape) == (T, W)
+    assert w is None or (w.dtype == torch.float32 and w.is_contiguous() and w.numel() == W)
+    vocab = 0
+    if table is not None:
+        assert table.is_contiguous() and table.dtype == dtype and table.shape[1] == W
+        assert tokens.dtype == torch.int64 and tokens.is_contiguous() and tokens.numel() == T
+        vocab = table.shape[0]
+    parts = split and dtype != torch.float32
+    h = None
+    if w is not None or parts:
+        h = torch.empty(2 * T if parts else T, W, dtype=dtype, device=x.device)
+    fp = list(f) + [None] * (2 - len(f))
+    call("sm_stream_rms", DT[dtype], x, int(bool(keep)), table, tokens, vocab, float(scale), y,
+         fp[0], fp[1], f2, float(coef), w, h, int(parts), T, W, eps)
+    return x if split and not parts else h
+
+
+def embed_rms(tokens: torch.Tensor, table: torch.Tensor, scale: float, out, eps: float):
+    """The start of a stream: x [T, W] fp32 = table[token] * ``scale`` and, in the table's dtype,
+    what ``out`` asks for: RMS norm with the fp32 weight ``out`` [W], SPLIT for the two 16-bit
+    parts [2 T, W] (fp32 model: x itself), None for nothing.  Returns (x, h)."""
+    x = torch.empty(tokens.shape[0], table.shape[1], dtype=torch.float32, device=table.device)
+    return x, _stream_rms(x, False, out, eps, table.dtype, tokens, table, scale)
+
+
+def residual_rms(x: torch.Tensor, y: torch.Tensor, out, eps: float):
+    """The stream ``x`` [T, W] fp32 takes a sublayer's output ``y`` (compute dtype) in place;
+    returns what ``out`` asks for (see ``embed_rms``)."""
+    return _stream_rms(x, True, out, eps, y.dtype, y=y)
+
+
+def parts_rms(parts: torch.Tensor, base: torch.Tensor, coef: float, out, eps: float, dtype):
+    """A new stream from a GEMM over the old one's parts: ``parts`` [T, W] or [2 T, W] fp32 (high
+    rows, then low rows) summed, plus ``coef`` * ``base`` [T, W] fp32.  Returns (x, h)."""
+    T, W = base.shape
+    x = torch.empty(T, W, dtype=torch.float32, device=base.device)
+    f = (parts,) if parts.shape[0] == T else (parts[:T], parts[T:])
+    return x, _stream_rms(x, False, out, eps, dtype, f=f, f2=base, coef=coef)
+
+
 # ---- a recurrence's read-out: group RMS norm and output gate ---------------------------------------
 # The fp32 row x is normed in ``groups`` equal parts (each by its own root mean square), weighted,
 # and gated by act(g) with act = SiLU or the sigmoid; the gate multiplies either before the norm or

@@ -202,6 +202,33 @@ def stretched_inv_freq(dims: int, base: float, scaling, device) -> torch.Tensor:
     return t
 
 
+def yarn_inv_freq(dims: int, base: float, scaling, device) -> Tuple[torch.Tensor, float]:
+    """YaRN: ([dims / 2] fp32 rotations per position, the factor cosine and sine carry).  Without
+    ``scaling`` the plain base^(-2i / dims) and 1.  With ``scaling`` = {factor, original, fast, slow}:
+    a dimension that turns more than ``fast`` times within ``original`` positions keeps its
+    frequency, one that turns less than ``slow`` times has it divided by ``factor``, between the two
+    the dimension's place decides (a linear ramp from floor of the first border to ceil of the
+    second, clamped to [0, dims - 1]); the factor is 0.1 ln(factor) + 1.  Computed in float64."""
+    if not scaling or not dims:
+        return interleaved_inv_freq(dims, base, device), 1.0
+    factor, orig, fast, slow = (float(scaling[k]) for k in ("factor", "original", "fast", "slow"))
+    amp = 0.1 * math.log(factor) + 1.0
+    key = ("yarn", int(dims), float(base), factor, orig, fast, slow, str(device))
+    t = _INV_FREQ.get(key)
+    if t is None:
+        def border(turns):             # the dimension that turns ``turns`` times in ``orig``
+            return dims * math.log(orig / (2.0 * math.pi * turns)) / (2.0 * math.log(float(base)))
+
+        lo, hi = max(math.floor(border(fast)), 0), min(math.ceil(border(slow)), dims - 1)
+        i = torch.arange(dims // 2, dtype=torch.float64)
+        ramp = torch.clamp((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+        f = torch.tensor([float(base) ** (-2.0 * k / dims) for k in range(dims // 2)],
+                         dtype=torch.float64)
+        t = (f / factor * ramp + f * (1.0 - ramp)).float().to(device)
+        _INV_FREQ[key] = t
+    return t, amp
+
+
 def rotate_interleaved_ref(x, positions, heads, head_stride, off, dims, inv_freq):
     T = x.shape[0]
     a = positions.float().view(T, 1, 1) * inv_freq.float().view(1, 1, -1)

@@ -1,12 +1,12 @@
 """Serving runner for stacks whose layers each name their own mixer (Gedatar, Dalavik,
-Fanopel, Foderax, Silonex): paged caches + per-sequence recurrent state.
+Fanopel, Foderax, Silonex, Tazulix): paged caches + per-sequence recurrent state.
 
-Five families share the runner, the segments, the block manager and the hipGraph decode; each
+Six families share the runner, the segments, the block manager and the hipGraph decode; each
 has its weights class (stacked projections, fp32 constants), its caches and its step function:
 Gedatar (``HybridWeights`` / ``HybridState`` / ``run_layers``, described next), Dalavik
 (``DalavikWeights`` / ``DalavikState``), Fanopel (``FanopelWeights`` / ``FanopelState``),
-Foderax (``FoderaxWeights`` / ``FoderaxState``) and Silonex (``SilonexWeights`` /
-``SilonexState``), further down.
+Foderax (``FoderaxWeights`` / ``FoderaxState``), Silonex (``SilonexWeights`` / ``SilonexState``)
+and Tazulix (``TazulixWeights`` / ``TazulixState``), further down.
 
 One step function for prefill chunks, decode rows and mixtures of both.  The rows of a step are
 cut into segments (``ops.segments.SegBatch``: one per chunk, one per decode row); per layer
@@ -43,14 +43,16 @@ import torch.nn.functional as F
 from ..models.config import ModelConfig
 from ..models.gedatar import DELTA_DECAY, DELTA_KEY_EPS
 from ..ops.attention import (chunk_sink_attention, diff_head_combine, head_norm_rotary_write,
-                             head_norm_write, latent_write, row_attention, row_norm_write,
-                             transposed_values_ok, write_key_cache)
+                             head_norm_write, latent_write, row_attention,
+                             row_norm_rotary_write, row_norm_write, transposed_values_ok,
+                             write_key_cache)
 from ..ops.conv import dyt_canon, short_conv
 from ..ops.embedding import embed_positions, embed_scaled, gated_token_slice, soft_cap
-from ..ops.moe import gated_act, moe, route_groups, route_topk, router_logits
-from ..ops.norm import (depth_mix_norm, dyt, dyt_residual, gated_rms_norm, group_rms_norm,
-                        group_rms_residual, hyper_mix, hyper_start, scaled_residual_layer_norm,
-                        weight_layer_norm)
+from ..ops.moe import (ClampedGate, gated_act, moe, route_groups, route_topk, router_logits,
+                       scaled_act)
+from ..ops.norm import (SPLIT, depth_mix_norm, dyt, dyt_residual, embed_rms, gated_rms_norm,
+                        group_rms_norm, group_rms_residual, hyper_mix, hyper_start, parts_rms,
+                        residual_rms, scaled_residual_layer_norm, weight_layer_norm)
 from ..ops.recurrent import delta_scan, head_scan, min_gru_scan, token_shift, wkv_scan
 from ..ops.rope import rotary_write, rotate_interleaved_
 from ..ops.segments import SegBatch, whole_sequences
@@ -190,6 +192,15 @@ def key_bytes_per_token(cfg: ModelConfig, dtype_bytes: int = 2) -> int:
                 a = cfg.layer_specs[i]["mixer"]["left"]
                 n += a["kv_heads"] * (a["dim"] + a["vdim"])
         return max(1, n * dtype_bytes)
+    if cfg.arch == "tazulix":                  # likewise
+        from ..models.tazulix import layer_runs
+
+        n = 0
+        for i in layer_runs(cfg):
+            m = cfg.layer_specs[i]["mixer"]
+            if cfg.layer_specs[i]["type"] == "attention":
+                n += m["kv_heads"] * (m["dim"] + m["vdim"])
+        return max(1, n * dtype_bytes)
     if cfg.arch == "dalavik":
         n = 0
         for L in cfg.layer_specs:
@@ -218,6 +229,12 @@ def state_bytes_per_slot(cfg: ModelConfig, dtype_bytes: int = 2) -> int:
             H, Dk, Dv, C, K = _silonex_state_sizes(cfg.layer_specs[i]["type"], m)
             n += 4 * H * Dk * Dv + dtype_bytes * C * (K - 1)
         return n
+    if cfg.arch == "tazulix":
+        from ..models.tazulix import layer_runs
+
+        ms = [cfg.layer_specs[i]["mixer"] for i in layer_runs(cfg)
+              if cfg.layer_specs[i]["type"] == "lightning"]
+        return 4 * sum(m["heads"] * m["dim"] * m["vdim"] for m in ms)
     n = 0
     for L in cfg.layer_specs:
         n += max(cfg.canon_taps - 1, 0) * cfg.hidden_size
@@ -1115,8 +1132,210 @@ def run_silonex_layers(w: SilonexWeights, st: SilonexState, tokens: torch.Tensor
     return h
 
 
+# ---- Tazulix: whole-projection normed attention beside lightning attention, looped with re-injection --
+#
+#   x = embed[token] * scale (fp32);  h = rms(x) * w_1                                  (embed_rms)
+#   p = W_in[:, width:] embed[token]    once per step: the looped passes' share of the embedding,
+#                                       fp32, without the scale (it joins as a factor)
+#   per pass of a layer (a looped layer: the same weights, its own caches and state)
+#   a loop's pass begins
+#       [hi ; lo] = the stream's two 16-bit parts       (by whoever wrote the stream: residual_rms)
+#       x  = W_in[:, :width] hi + W_in[:, :width] lo + scale * p;  h = rms(x) * w_1
+#                                       one GEMM over 2 T rows, fp32 result             (parts_rms)
+#   attention
+#       z  = [W_q ; W_k ; W_v] h + b    one GEMM
+#       q, k normed over their whole projections and turned; k, v to their caches
+#                                                                          (row_norm_rotary_write)
+#       y  = W_o row_attention(z's q)
+#   lightning
+#       z  = [W_q ; W_k ; W_v ; W_g] h;  r = head_scan(constant decays, silu on q, k, v)
+#       y  = W_o (rms(r) w sigmoid(g))                                      (gated_rms_norm)
+#   x += y;  h = rms(x) * w_2                                               (residual_rms)
+#   dense:    y = W_down relu(W_up h)^2
+#   experts:  r = route_groups(W_r h in fp32: sigmoids as they are, the top ones)
+#             y = [W_down_e | W_down_s] act([gate | up] of every expert, times r | of the shared one)
+#                 with the routing weight on the gate and up values (moe, weigh="input")
+#   x += y;  h = rms(x) * w_1 of the next pass, or the next loop pass's two parts
+#   logits = rms(x) * w_final through the head       fp32 product of the 16-bit operands
+#
+# fp32: the stream and what joins it, norms, angles, scores, softmax, decays, states, read-outs, the
+# router, logits; model dtype: GEMMs and what they store.
+@dataclass
+class TazulixLayerW:
+    kind: str                       # attention | lightning
+    m: dict                         # the mixer's sizes and constants
+    norm1: torch.Tensor
+    w: Dict[str, torch.Tensor] = field(default_factory=dict)
+    cols: List[int] = field(default_factory=list)     # lightning: first columns of q, k, v, g
+    amp: float = 1.0                # attention: factor on cosine and sine
+    rot_dims: int = 0
+    ff: Optional[dict] = None       # norm, down; dense: up, ff; experts: gu, router, E, top, ff, ...
+
+
+class TazulixWeights:
+    """Inference weights of a TazulixForCausalLM: projections that share an input (and their biases)
+    are stacked into one GEMM, the experts' [gate | up] rows and the shared expert's into another,
+    their down projections side by side; the loop's input projection is kept as its two halves;
+    norms and decays are fp32.  ``runs`` lists the layer of every pass, ``starts`` whether a loop's
+    pass begins with it: caches and state are kept per pass."""
+
+    def __init__(self, model, tp_rank: int = 0, tp_size: int = 1):
+        if tp_size != 1:
+            raise NotImplementedError("Tazulix models are served at tensor-parallel size 1")
+        from ..models.tazulix import GATE_SLOPE, UP_SHIFT, layer_runs, pass_starts, rotary
+        from ..ops.rope import yarn_inv_freq
+
+        cfg: ModelConfig = model.config
+        self.cfg = cfg
+        t = model.tensor
+        f32 = lambda n: t(n).detach().float().contiguous()  # noqa: E731
+        self.dtype = dt = t("embed").dtype
+        dev = t("embed").device
+        self.embed = t("embed").detach()
+        self.lm_head = t("head").detach()
+        self.final = f32("final.norm")
+        self.vocab_shard = cfg.vocab_size
+        self.scale = float(cfg.embedding_scale)
+        self.runs = layer_runs(cfg)
+        self.starts = pass_starts(cfg)
+        self.layers: List[TazulixLayerW] = []
+        with torch.no_grad():
+            self.loop_x = self.loop_e = None
+            if any(self.starts):
+                W = cfg.hidden_size
+                self.loop_x = t("loop.in")[:, :W].contiguous()
+                self.loop_e = t("loop.in")[:, W:].contiguous()
+            for i, spec in enumerate(cfg.layer_specs):
+                p, m, f = f"l{i}.", spec["mixer"], spec.get("mlp")
+                x, y = p + "mix.", p + "mlp."
+                L = TazulixLayerW(spec["type"], m, f32(p + "norm1"))
+                if L.kind == "attention":
+                    L.w["in"] = _pad_rows([t(x + n) for n in "qkv"], dt, dev)
+                    b = torch.cat([t(x + n + ".b") for n in "qkv"], 0)
+                    L.w["in_b"] = torch.cat([b, b.new_zeros(L.w["in"].shape[0] - b.shape[0])])
+                    L.w["q.norm"], L.w["k.norm"] = f32(x + "q.norm"), f32(x + "k.norm")
+                    L.rot_dims, base, scaling = rotary(m)
+                    L.w["inv_freq"], L.amp = yarn_inv_freq(L.rot_dims, base, scaling, dev)
+                else:
+                    L.w["in"], L.cols = _stack_rows([[t(x + n)] for n in "qkvg"], dt, dev)
+                    decay = torch.tensor([float(d) for d in m["decay"]], dtype=torch.float64)
+                    L.w["log_decay"] = torch.log(decay).clamp(min=-1e4).float().to(dev)
+                    L.w["norm"] = f32(x + "norm")
+                L.w["o"] = t(x + "o").detach()
+                if f and f["kind"] == "dense":
+                    L.ff = dict(E=0, ff=int(f["ff"]), up=t(y + "up").detach(),
+                                down=t(y + "down").detach(), norm=f32(p + "norm2"))
+                elif f:
+                    E, sh = int(f["router"]["experts"]), f.get("shared")
+                    names = [y + f"e{e}." for e in range(E)] + ([y + "shared."] if sh else [])
+                    limit = float(f["expert"]["limit"])
+                    L.ff = dict(E=E, top=int(f["router"]["top"]), ff=int(f["expert"]["ff"]),
+                                ffs=int(sh["ff"]) if sh else 0, norm=f32(p + "norm2"),
+                                router=t(y + "router").detach(),
+                                gu=torch.cat([t(n + s) for n in names for s in ("gate", "up")],
+                                             0).contiguous(),
+                                down=torch.cat([t(n + "down") for n in names], 1).contiguous(),
+                                act=ClampedGate(limit, float(sh["limit"]) if sh else limit,
+                                                GATE_SLOPE, UP_SHIFT))
+                self.layers.append(L)
+
+    def new_state(self, slots: int, num_blocks: int, block_size: int, device):
+        return TazulixState(self, slots, num_blocks, block_size, device)
+
+    def run_layers(self, st, tokens, seg, observe=None) -> torch.Tensor:
+        return run_tazulix_layers(self, st, tokens, seg, observe)
+
+    def head(self, x: torch.Tensor) -> torch.Tensor:
+        h = group_rms_norm(x, self.final, 1, self.cfg.rms_norm_eps, self.dtype)
+        return router_logits(h, self.lm_head)     # fp32 logits from the 16-bit (or fp32) operands
+
+
+class TazulixState:
+    """Caches and state of a Tazulix model, one set per PASS of a layer (``TazulixWeights.runs``).
+    Paged through the engine's block manager: turned keys and values of every attention pass.  Per
+    state slot (+ one spare for graph padding rows): the fp32 matrix state [slots + 1, heads, key,
+    value] of every lightning pass."""
+
+    def __init__(self, w: TazulixWeights, slots: int, num_blocks: int, block_size: int, device):
+        self.slots = slots
+        self.spare = slots
+        kw = dict(dtype=w.dtype, device=device)
+        self.k: List[Optional[torch.Tensor]] = []
+        self.v: List[Optional[torch.Tensor]] = []
+        self.S: List[Optional[torch.Tensor]] = []
+        for i in w.runs:
+            L = w.layers[i]
+            m, att = L.m, L.kind == "attention"
+            page = (num_blocks, block_size)
+            self.k.append(torch.zeros(*page, m["kv_heads"], m["dim"], **kw) if att else None)
+            self.v.append(torch.zeros(*page, m["kv_heads"], m["vdim"], **kw) if att else None)
+            self.S.append(None if att else torch.zeros(slots + 1, m["heads"], m["dim"], m["vdim"],
+                                                       dtype=torch.float32, device=device))
+
+
+def _tazulix_mixer(L: TazulixLayerW, w: TazulixWeights, st: TazulixState, n: int, h, seg):
+    """Pass ``n``'s mixer on its normed input h [T, W]."""
+    m, dt, eps = L.m, w.dtype, w.cfg.rms_norm_eps
+    T = h.shape[0]
+    H, D, Dv = m["heads"], m["dim"], m["vdim"]
+    if L.kind == "attention":
+        G = m["kv_heads"]
+        z = F.linear(h, L.w["in"], L.w["in_b"])
+        row_norm_rotary_write(z, L.w["q.norm"], L.w["k.norm"], seg.positions, seg.cache_slots,
+                              st.k[n], st.v[n], H, G, D, Dv, L.rot_dims, L.w["inv_freq"], L.amp,
+                              eps)
+        o = torch.empty(T, H, Dv, dtype=dt, device=h.device)
+        row_attention(z[:, :H * D].view(T, H, D), None, st.k[n], st.v[n], Dv, o, seg, H, G,
+                      float(m["scale"]))
+        return F.linear(o.view(T, H * Dv), L.w["o"])
+    z = F.linear(h, L.w["in"])
+    q0, k0, v0, g0 = L.cols
+    y = head_scan(z[:, q0:q0 + H * D], z[:, k0:k0 + H * D], z[:, v0:v0 + H * Dv], st.S[n], seg, H,
+                  D, Dv, L.w["log_decay"], silu_in=True)
+    y = gated_rms_norm(y, z[:, g0:g0 + H * Dv], L.w["norm"], 1, eps, "sigmoid", False)
+    return F.linear(y, L.w["o"])
+
+
+def _tazulix_ff(f: dict, h) -> torch.Tensor:
+    if not f["E"]:
+        return F.linear(scaled_act(F.linear(h, f["up"]), None, 0, 0, f["ff"], "relu2"), f["down"])
+    # the router in fp32, on the (possibly 16-bit rounded) normed row
+    r = route_groups(router_logits(h, f["router"]), None, f["top"], 1, 1, normalize=False)
+    return moe(h, r, f["gu"], f["down"], f["E"], f["top"], f["ff"], f["ffs"], f["act"],
+               weigh="input")
+
+
+def run_tazulix_layers(w: TazulixWeights, st: TazulixState, tokens: torch.Tensor, seg: SegBatch,
+                       observe=None) -> torch.Tensor:
+    """The step function: token ids [T] + their segments -> the fp32 residual stream [T, W] after
+    the last pass; caches and state in ``st`` move on by the step's rows.  ``observe`` is called
+    with every pass's number and the stream after it."""
+    eps, n_runs = w.cfg.rms_norm_eps, len(w.runs)
+
+    def want(n):
+        """What pass ``n`` reads: its first norm's weight, or the stream's parts when a loop's pass
+        begins there, or nothing after the last."""
+        return None if n == n_runs else SPLIT if w.starts[n] else w.layers[w.runs[n]].norm1
+
+    p = router_logits(F.embedding(tokens, w.embed), w.loop_e) if any(w.starts) else None
+    x, h = embed_rms(tokens, w.embed, w.scale, want(0), eps)
+    for n, i in enumerate(w.runs):
+        L = w.layers[i]
+        if w.starts[n]:
+            x, h = parts_rms(router_logits(h, w.loop_x), p, w.scale, L.norm1, eps, w.dtype)
+        y = _tazulix_mixer(L, w, st, n, h, seg)
+        if L.ff is None:
+            h = residual_rms(x, y, want(n + 1), eps)
+        else:
+            h = residual_rms(x, y, L.ff["norm"], eps)
+            h = residual_rms(x, _tazulix_ff(L.ff, h), want(n + 1), eps)
+        if observe is not None:
+            observe(n, x)
+    return x
+
+
 WEIGHTS = {"gedatar": HybridWeights, "dalavik": DalavikWeights, "fanopel": FanopelWeights,
-           "foderax": FoderaxWeights, "silonex": SilonexWeights}
+           "foderax": FoderaxWeights, "silonex": SilonexWeights, "tazulix": TazulixWeights}
 
 
 class HybridRunner(ModelRunner):
