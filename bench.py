@@ -495,7 +495,7 @@ def main():
                          "per-layer-mixer design (--hybrid_family) beside Llama at equal size, "
                          "one GPU (lumen/bench/hybrid_bench.py)")
     ap.add_argument("--hybrid_family", default="gedatar",
-                    choices=["gedatar", "dalavik", "fanopel", "foderax", "silonex"])
+                    choices=["gedatar", "dalavik", "fanopel", "foderax", "silonex", "tazulix"])
     ap.add_argument("--hybrid_only", action="store_true",
                     help="with --hybrid: run the family alone, without the models beside it "
                          "(a kernel trace of one design)")

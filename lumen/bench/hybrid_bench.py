@@ -1,12 +1,13 @@
 """Prefill / decode throughput of a per-layer-mixer design (Gedatar, Dalavik, Fanopel, Foderax,
-Silonex) beside Llama at equal size.
+Silonex, Tazulix) beside Llama at equal size.
 
-``python bench.py --hybrid [--hybrid_family dalavik|fanopel|foderax|silonex]`` (one GPU).  Fanopel also
-runs beside the closest design the framework already had: a Gedatar stack of attention layers
+``python bench.py --hybrid [--hybrid_family dalavik|fanopel|foderax|silonex|tazulix]`` (one GPU).
+Fanopel also runs beside the closest design the framework already had: a Gedatar stack of attention layers
 (keys as values) with routed experts of the same shapes; Foderax beside Dalavik (latent and
 grouped-query attention through the same row kernels) and Fanopel (experts of the same shapes);
 Silonex beside Gedatar (matrix-state recurrences of the same head sizes, dense feed-forwards) and
-Fanopel (window attention through the same kernels).  All models get random weights of layer shapes
+Fanopel (window attention through the same kernels); Tazulix beside Silonex (lightning attention and
+the scan kernels) and Fanopel (whole-projection norms, sigmoid-routed experts).  All models get random weights of layer shapes
 that resemble real models (width 2048 / 4096, head size 128 / 64, FFN 2.75 x width, vocab 32000), the
 same depth, and run the same forced-token workload through the serving engine
 (``lumen.serve.trace.TraceReplay``: the engine's input builder, block manager, state slots,
@@ -164,6 +165,35 @@ def silonex_config(width: int, depth_groups: int = 1):
                        name=f"silonex-w{W}", layer_specs=layers)
 
 
+def tazulix_config(width: int, depth_groups: int = 1):
+    """Per group of four: lightning attention with heads of 128 and a dense squared-ReLU FFN of 2.75 x
+    width, then attention (heads of 128, one key head per four query heads, YaRN on the whole head),
+    lightning and attention with 16 gated experts of FFN width 2.75 / 4 x model width, top 3, and a
+    shared one of the same width: the active FFN width equals the dense 2.75 x width.  One pass
+    through a loop over the middle layers: its input projection runs, the depth stays comparable."""
+    from ..models.config import ModelConfig
+
+    W = width
+    H = W // 128
+    ffe = int(2.75 * W) // 4
+    moe = {"kind": "moe", "router": {"experts": 16, "top": 3},
+           "expert": {"ff": ffe, "limit": 7.0}, "shared": {"ff": ffe, "limit": 7.0}}
+    att = {"type": "attention", "mlp": moe, "mixer": {
+        "heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+        "rot": {"base": 500000.0, "dims": 128,
+                "scaling": {"factor": 8.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}}
+    lin = {"heads": H, "dim": 128, "vdim": 128,
+           "decay": [1.0 - 2.0 ** (-2 - 6 * i / H) for i in range(H)]}
+    layers = [{"type": "lightning", "mlp": {"kind": "dense", "ff": int(2.75 * W)}, "mixer": lin},
+              att, {"type": "lightning", "mlp": moe, "mixer": lin}, att] * depth_groups
+    return ModelConfig(arch="tazulix", vocab_size=32000, hidden_size=W,
+                       num_hidden_layers=len(layers), rms_norm_eps=1e-6,
+                       embedding_scale=float(W) ** 0.5, loop={"start": 1, "stop": 3, "times": 1},
+                       intermediate_size=0, num_attention_heads=0, num_key_value_heads=0,
+                       max_position_embeddings=1 << 20, eos_token_id=-1,
+                       name=f"tazulix-w{W}", layer_specs=layers)
+
+
 def gedatar_attention_moe_config(width: int, depth: int = 4):
     """The closest older design at Fanopel's shapes: Gedatar attention layers (keys as values,
     chunk mask of 1024) with 16 gated experts of the same FFN width, top 4, no shared expert."""
@@ -257,7 +287,8 @@ def run_hybrid_bench(args) -> list:
     rows = []
     family = getattr(args, "hybrid_family", "gedatar")
     make = {"gedatar": gedatar_config, "dalavik": dalavik_config, "fanopel": fanopel_config,
-            "foderax": foderax_config, "silonex": silonex_config}[family]
+            "foderax": foderax_config, "silonex": silonex_config,
+            "tazulix": tazulix_config}[family]
     for width in [int(w) for w in str(args.hybrid_widths).split(",")]:
         gcfg = make(width)
         beside = [llama_config(width, gcfg.num_hidden_layers)]
@@ -267,6 +298,8 @@ def run_hybrid_bench(args) -> list:
             beside = [dalavik_config(width), fanopel_config(width, gcfg.num_hidden_layers)] + beside
         if family == "silonex":
             beside = [gedatar_config(width), fanopel_config(width, gcfg.num_hidden_layers)] + beside
+        if family == "tazulix":
+            beside = [silonex_config(width), fanopel_config(width, gcfg.num_hidden_layers)] + beside
         if getattr(args, "hybrid_only", False):
             beside = []
         for cfg in [gcfg] + beside:
@@ -290,7 +323,8 @@ def run_hybrid_bench(args) -> list:
             gd = by[(w, b, "gedatar")]
             row["prefill_vs_gedatar"] = round(r["prefill_tok_s"] / gd["prefill_tok_s"], 3)
             row["decode_vs_gedatar"] = round(r["decode_tok_s"] / gd["decode_tok_s"], 3)
-        others = {"foderax": ("dalavik", "fanopel"), "silonex": ("gedatar", "fanopel")}
+        others = {"foderax": ("dalavik", "fanopel"), "silonex": ("gedatar", "fanopel"),
+                  "tazulix": ("silonex", "fanopel")}
         if family in others:
             for other in others[family]:
                 o = by[(w, b, other)]
