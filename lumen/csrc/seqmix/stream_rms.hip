@@ -7,7 +7,8 @@
 //                     or its two 16-bit parts hi = round(x'), lo = round(x' - hi)   (split): a
 //                     GEMM over both keeps about 16 bits of the stream's mantissa
 //                     or nothing but x' itself
-//                 x, f0, f1, f2 are fp32; y and the embedding table are in the compute dtype.
+//                 x, f0, f1, f2 are fp32; y and the embedding table are in the compute dtype.  With
+//                 `rows` the token's table row is also copied out as it is (a GEMM's operand).
 //
 // One workgroup per row, four channels per lane; the new row stays in LDS between the sum of squares
 // and the output.
@@ -22,7 +23,7 @@ constexpr int kThreads = 256;
 template <typename T>
 struct StreamArgs {
   float* x; int keep;                                   // keep: x is one of the addends
-  const T* table; const long long* tokens; int vocab; float scale;
+  const T* table; const long long* tokens; int vocab; float scale; T* rows;
   const T* y;
   const float* f0; const float* f1; const float* f2; float coef;
   const float* w; T* h; int split;
@@ -68,7 +69,13 @@ __global__ void __launch_bounds__(kThreads) stream_rms_kernel(const StreamArgs<T
 #pragma unroll
       for (int e = 0; e < V; ++e) v[e] = 0.f;
     }
-    if (er != nullptr) add_n<T, V>(er + c, a.scale, v);
+    if (er != nullptr) {
+      float ev[V];
+      load_n<T, V>(er + c, ev);
+      if (a.rows != nullptr) store_n<T, V>(a.rows + base + c, ev);      // exact: the table's own values
+#pragma unroll
+      for (int e = 0; e < V; ++e) v[e] += a.scale * ev[e];
+    }
     if (a.y != nullptr) add_n<T, V>(a.y + base + c, 1.f, v);
     if (a.f0 != nullptr) add_n<float, V>(a.f0 + base + c, 1.f, v);
     if (a.f1 != nullptr) add_n<float, V>(a.f1 + base + c, 1.f, v);
@@ -109,21 +116,22 @@ extern "C" {
 // x fp32 [rows][W] (written; read with keep).  h [rows][W], or with split [2 rows][W]: the high parts
 // of all rows, then the low parts.
 hipError_t sm_stream_rms(int dt, float* x, int keep, const void* table, const long long* tokens,
-                         int vocab, float scale, const void* y, const float* f0, const float* f1,
-                         const float* f2, float coef, const float* w, void* h, int split, int rows,
-                         int W, float eps, hipStream_t st) {
+                         int vocab, float scale, void* table_rows, const void* y, const float* f0,
+                         const float* f1, const float* f2, float coef, const float* w, void* h,
+                         int split, int rows, int W, float eps, hipStream_t st) {
   if (rows == 0) return hipSuccess;
   if (W < 1 || (w && (size_t)W * sizeof(float) > 65536 - 64)) return hipErrorInvalidValue;
-  if (!x || (table && (!tokens || vocab < 1)) || (w && split) || ((w || split) && !h))
+  if (!x || (table && (!tokens || vocab < 1)) || (table_rows && !table) || (w && split) ||
+      ((w || split) && !h))
     return hipErrorInvalidValue;
   const auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
-  const bool vec = W % 4 == 0 && al(x) && al(table) && al(y) && al(f0) && al(f1) && al(f2) &&
-                   al(w) && al(h);
+  const bool vec = W % 4 == 0 && al(x) && al(table) && al(table_rows) && al(y) && al(f0) &&
+                   al(f1) && al(f2) && al(w) && al(h);
   const size_t lds = w != nullptr ? (size_t)W * sizeof(float) : 0;
 #define CALL(T)                                                                                   \
   {                                                                                               \
-    StreamArgs<T> a{x, keep, (const T*)table, tokens, vocab, scale, (const T*)y, f0, f1, f2, coef, \
-                    w, (T*)h, split, (long long)rows * W, W, eps};                                \
+    StreamArgs<T> a{x, keep, (const T*)table, tokens, vocab, scale, (T*)table_rows, (const T*)y,  \
+                    f0, f1, f2, coef, w, (T*)h, split, (long long)rows * W, W, eps};              \
     if (vec) stream_rms_kernel<T, 4><<<rows, kThreads, lds, st>>>(a);                             \
     else stream_rms_kernel<T, 1><<<rows, kThreads, lds, st>>>(a);                                 \
   }

@@ -57,7 +57,7 @@ SIGNATURES = {
     "sm_hyper_mix": "i" "pppi" "ppppf" "ppp" "ppf" "pp" "iiii",
     "sm_head_norm_rotary": "ipl" "ppppppp" "iiiiiiif",
     "sm_row_norm_rotary": "ipl" "ppppppp" "iiiiii" "ff",
-    "sm_stream_rms": "ipi" "ppif" "p" "pppf" "ppi" "iif",
+    "sm_stream_rms": "ipi" "ppifp" "p" "pppf" "ppi" "iif",
     "sm_head_scan_chunk": "ii" "plplplplpl" "pppp" "pp" "ppp" "iiiiiiff",
     "sm_head_scan_step": "ii" "plplplplpl" "pppp" "pp" "ppp" "iiiiiiff",
     "sm_short_conv": "iplpppp" "pppp" "iii",

@@ -246,8 +246,8 @@ def rms_norm_rows_ref(x, w, eps, out_dtype):
     return (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
 
 
-def _stream_rms(x, keep, out, eps, dtype, tokens=None, table=None, scale=1.0, y=None, f=(),
-                f2=None, coef=0.0):
+def _stream_rms(x, keep, out, eps, dtype, tokens=None, table=None, scale=1.0, rows=None, y=None,
+                f=(), f2=None, coef=0.0):
     """The new stream in ``x`` [T, W]; ``out``: a norm weight, SPLIT or None -> h, parts or None."""
     from ._seqmix import DT, call, use_seqmix
 
@@ -257,6 +257,8 @@ def _stream_rms(x, keep, out, eps, dtype, tokens=None, table=None, scale=1.0, y=
         v = x if keep else torch.zeros_like(x)
         if table is not None:
             v = v + table[tokens].float() * scale
+            if rows is not None:
+                rows.copy_(table[tokens])
         for p in ([y] if y is not None else []) + list(f):
             v = v + p.float()
         if f2 is not None:
@@ -284,17 +286,21 @@ def _stream_rms(x, keep, out, eps, dtype, tokens=None, table=None, scale=1.0, y=
     if w is not None or parts:
         h = torch.empty(2 * T if parts else T, W, dtype=dtype, device=x.device)
     fp = list(f) + [None] * (2 - len(f))
-    call("sm_stream_rms", DT[dtype], x, int(bool(keep)), table, tokens, vocab, float(scale), y,
-         fp[0], fp[1], f2, float(coef), w, h, int(parts), T, W, eps)
+    call("sm_stream_rms", DT[dtype], x, int(bool(keep)), table, tokens, vocab, float(scale), rows,
+         y, fp[0], fp[1], f2, float(coef), w, h, int(parts), T, W, eps)
     return x if split and not parts else h
 
 
-def embed_rms(tokens: torch.Tensor, table: torch.Tensor, scale: float, out, eps: float):
+def embed_rms(tokens: torch.Tensor, table: torch.Tensor, scale: float, out, eps: float,
+              rows: bool = False):
     """The start of a stream: x [T, W] fp32 = table[token] * ``scale`` and, in the table's dtype,
     what ``out`` asks for: RMS norm with the fp32 weight ``out`` [W], SPLIT for the two 16-bit
-    parts [2 T, W] (fp32 model: x itself), None for nothing.  Returns (x, h)."""
-    x = torch.empty(tokens.shape[0], table.shape[1], dtype=torch.float32, device=table.device)
-    return x, _stream_rms(x, False, out, eps, table.dtype, tokens, table, scale)
+    parts [2 T, W] (fp32 model: x itself), None for nothing.  Returns (x, h, e), e being the table's
+    rows as they are when ``rows`` asks for them, else None."""
+    shape = (tokens.shape[0], table.shape[1])
+    x = torch.empty(shape, dtype=torch.float32, device=table.device)
+    e = torch.empty(shape, dtype=table.dtype, device=table.device) if rows else None
+    return x, _stream_rms(x, False, out, eps, table.dtype, tokens, table, scale, e), e
 
 
 def residual_rms(x: torch.Tensor, y: torch.Tensor, out, eps: float):

@@ -1317,8 +1317,9 @@ def run_tazulix_layers(w: TazulixWeights, st: TazulixState, tokens: torch.Tensor
         begins there, or nothing after the last."""
         return None if n == n_runs else SPLIT if w.starts[n] else w.layers[w.runs[n]].norm1
 
-    p = router_logits(F.embedding(tokens, w.embed), w.loop_e) if any(w.starts) else None
-    x, h = embed_rms(tokens, w.embed, w.scale, want(0), eps)
+    looped = any(w.starts)
+    x, h, e = embed_rms(tokens, w.embed, w.scale, want(0), eps, rows=looped)
+    p = router_logits(e, w.loop_e) if looped else None
     for n, i in enumerate(w.runs):
         L = w.layers[i]
         if w.starts[n]:

@@ -126,7 +126,8 @@ def test_stream_start_and_residual(device, dtype, W):
     table = rnd(V, W, seed=1, dtype=dtype, device=device, scale=0.1)
     toks = torch.tensor([0, 32, 5, 5, 17, 1, 9], device=device)
     w = rnd(W, seed=4, device=device) + 1.0
-    x, h = embed_rms(toks, table, 8.5, w, 1e-2)
+    x, h, e = embed_rms(toks, table, 8.5, w, 1e-2)
+    assert e is None
     xd = f64(table)[toks.cpu()] * 8.5
     assert x.dtype == torch.float32 and h.dtype == dtype
     close(x, xd, torch.float32)
@@ -157,7 +158,8 @@ def test_stream_through_its_own_projection(device, dtype, W):
     base = mm(table[toks], B)
     for start in (True, False):
         if start:
-            x, parts = embed_rms(toks, table, 3.0, SPLIT, 1e-5)
+            x, parts, e = embed_rms(toks, table, 3.0, SPLIT, 1e-5, rows=True)
+            assert torch.equal(e, table[toks])
         else:
             parts = residual_rms(x, rnd(T, W, seed=6, dtype=dtype, device=device), SPLIT, 1e-5)
         xd = f64(x)
