@@ -274,13 +274,21 @@ def moe_grouped_mm(h, wts, gu_w, down_w, E: int, top: int, ff: int, ffs: int, ac
     return out.to(h.dtype)
 
 
-# When the grouped form pays.  Measured on MI355X (bf16, width 2048, 16 experts of 1408, top 4):
-# the two stacked GEMMs of the dense form run at ~850 TFLOP/s, the grouped GEMMs at ~300, and
-# sorting the (row, expert) pairs costs ~0.4 ms per layer whatever the size.  The grouped form does
+# When the grouped form pays.  Measured on MI355X (bf16, 16 experts, widths 1024 - 4096, 512 - 16384
+# rows): the two stacked GEMMs of the dense form run at ~850 TFLOP/s, the grouped GEMMs at ~300, and
+# sorting the (row, expert) pairs costs ~0.4 - 0.8 ms per layer whatever the size.  The grouped form does
 # top / E of the dense form's FLOPs at about a third of its rate, so it needs E > 3 top to save
-# anything, and enough rows for the saving to cover the sorting.
+# anything, and enough products saved in the experts' first GEMM to cover the sorting: the two forms
+# take the same time between 90 and 170 G multiply-adds at every size (inside a model the dense form's
+# two launches also hide better), so the grouped one is taken above that.
 GROUPED_RATE_RATIO = 3
-GROUPED_MIN_SAVING = 32768          # rows x (E - GROUPED_RATE_RATIO * top)
+GROUPED_MIN_SAVING = 180e9          # rows x (E - GROUPED_RATE_RATIO * top) x an expert's [k ff, W]
+
+
+def grouped_pays(rows: int, E: int, top: int, expert_weights: int) -> bool:
+    """Do ``rows`` rows save enough by visiting only their chosen experts (``expert_weights``:
+    elements of one expert's first projection)?"""
+    return rows * (E - GROUPED_RATE_RATIO * top) * expert_weights >= GROUPED_MIN_SAVING
 
 
 def moe(h, wts, gu_w, down_w, E: int, top: int, ff: int, ffs: int, act="silu",
@@ -290,8 +298,7 @@ def moe(h, wts, gu_w, down_w, E: int, top: int, ff: int, ffs: int, act="silu",
     expert in ``gu_w`` (``act`` also a ``ClampedGate``); else W_down act(W_up h) with the up rows
     alone.  ``weigh`` = "input": an expert sees its weight times h instead of weighing in with its
     output (gated experts)."""
-    spare = E - GROUPED_RATE_RATIO * top
-    grouped = (spare > 0 and h.shape[0] * spare >= GROUPED_MIN_SAVING
+    grouped = (grouped_pays(h.shape[0], E, top, (2 if gated else 1) * ff * h.shape[1])
                and not (h.is_cuda and torch.cuda.is_current_stream_capturing()))
     if grouped and grouped_mm_ok(h, ff):
         return moe_grouped_mm(h, wts, gu_w, down_w, E, top, ff, ffs, act, gated, weigh)

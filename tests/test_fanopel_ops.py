@@ -436,12 +436,14 @@ def test_router_logits_are_fp32_sums_of_exact_products(device, dtype):
 @pytest.mark.parametrize("dtype", [torch.bfloat16, torch.float16])
 @pytest.mark.parametrize("E,top,n,keep,ff,W,T", [(40, 2, 1, 1, 16, 64, 1000), (64, 4, 8, 2, 8, 40, 1200),
                                                  (33, 1, 1, 1, 24, 128, 1100)])
-def test_grouped_gemm_form_with_idle_experts(dtype, E, top, n, keep, ff, W, T):
+def test_grouped_gemm_form_with_idle_experts(dtype, E, top, n, keep, ff, W, T, monkeypatch):
     """The sync-free grouped form as ``moe`` picks it for many experts and few chosen: a correction
     of -10 keeps a third of the experts from ever being chosen, so their groups are empty; one
     expert takes every row."""
+    import lumen.ops.moe as moe_ops
     from lumen.ops.moe import moe
 
+    monkeypatch.setattr(moe_ops, "GROUPED_MIN_SAVING", 1)      # small shapes take the grouped GEMM
     device = "cuda"
     h = rnd(T, W, seed=70, dtype=dtype, device=device)
     w = {"m.router": rnd(E, W, seed=71, scale=0.5), "m.correction": rnd(E, seed=72, scale=0.2)}
@@ -458,6 +460,6 @@ def test_grouped_gemm_form_with_idle_experts(dtype, E, top, n, keep, ff, W, T):
     r = route_groups(h.float() @ w["m.router"].to(device).t(), w["m.correction"].to(device), top, n,
                      keep, 1.3)
     assert int((r[:, ::3] > 0).sum()) == 0 and bool((r[:, 1] > 0).all())
-    assert grouped_mm_ok(h, ff) and T * (E - 3 * top) >= 32768     # moe() takes the grouped GEMM
+    assert grouped_mm_ok(h, ff) and moe_ops.grouped_pays(T, E, top, ff * W)
     close(moe(h, r, up, down, E, top, ff, 0, "relu2", gated=False), want, dtype)
     close(moe_grouped_mm(h, r, up, down, E, top, ff, 0, "relu2", gated=False), want, dtype)

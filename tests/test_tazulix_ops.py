@@ -275,12 +275,23 @@ def test_experts_of_weighted_inputs_match_oracle(device, dtype, E, top, ff, ffs)
     assert float((f64(off) - want).abs().max()) > 0.1
 
 
+def test_grouped_form_is_chosen_by_what_it_saves():
+    from lumen.ops.moe import grouped_pays
+
+    big = 2 * 2816 * 4096
+    assert grouped_pays(2048, 16, 3, big) and not grouped_pays(8, 16, 3, big)
+    assert not grouped_pays(1 << 20, 16, 6, big)               # 3 top > E: nothing to save
+    assert not grouped_pays(4096, 16, 3, 2 * 704 * 1024)       # narrow layers: sorting costs more
+
+
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("E,top,ff,ffs,T", [(40, 2, 16, 24, 1000), (33, 1, 24, 0, 1100)])
-def test_grouped_experts_of_weighted_inputs(dtype, E, top, ff, ffs, T):
-    """The sizes at which ``moe`` leaves the dense form: the grouped GEMM in 16 bits, per-expert GEMMs
-    in fp32."""
+def test_grouped_experts_of_weighted_inputs(dtype, E, top, ff, ffs, T, monkeypatch):
+    """``moe`` leaving the dense form: the grouped GEMM in 16 bits, per-expert GEMMs in fp32."""
+    import lumen.ops.moe as moe_ops
+
+    monkeypatch.setattr(moe_ops, "GROUPED_MIN_SAVING", 1)
     W = 64
     h = rnd(T, W, seed=62, dtype=dtype, device="cuda")
     w, gu, down = _experts(E, ff, ffs, W, dtype, "cuda")
@@ -289,7 +300,7 @@ def test_grouped_experts_of_weighted_inputs(dtype, E, top, ff, ffs, T):
         f["shared"] = {"ff": ffs, "limit": 1.6}
     want = ref.moe_ff(f64(h), {k: v.to(F64) for k, v in w.items()}, "m.", f)
     r = route_groups(h.float() @ w["m.router"].float().cuda().t(), None, top, 1, 1, normalize=False)
-    assert T * (E - 3 * top) >= 32768
+    assert moe_ops.grouped_pays(T, E, top, 2 * ff * W)
     close(moe(h, r, gu, down, E, top, ff, ffs, GATE, weigh="input"), want, dtype)
 
 
