@@ -78,7 +78,7 @@ CONFIGS = {
     # head sizes 64 and 128 (the matrix-core attention's shapes), values twice as wide as keys, wide
     # states, the whole stack looped, one expert of many
     "wide": lambda: _cfg("wide", 200, 128, 11.3, {"start": 0, "stop": 3, "times": 2}, 1e-5, [
-        _att(4, 1, 64, 64, 32, _moe(12, 1, 48, 64), base=500000.0, scale=0.125),
+        _att(4, 1, 64, 64, 32, _moe(12, 1, 48, 64), base=500000.0, scale=0.13),
         _lin(2, 128, 64, [0.8, 0.995], _moe(8, 4, 32, 32, 3.0, 0.6)),
         _att(2, 2, 64, 128, 64, _ff(96), base=10000.0, scale=0.12)]),
 }
